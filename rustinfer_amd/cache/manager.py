@@ -2,12 +2,12 @@
 and slots of fixed-size state.
 
 Layers are sorted into *groups* by what they need: every position's keys and values, or
-only a window of them, with a given number of heads and head size.  A group has pages of
+only a window or a chunk of them, with a given number of heads and head size.  A group has pages of
 its own (one pool for all its layers: page ``p`` means the same tokens in each of them,
 as in the reference where one block id addresses every layer,
 crates/infer-worker/src/application/runtime/mod.rs:311-332) and a block table for each
 request.  Pages are taken when a request's tokens first need them, given back when the
-request is released or, in a windowed group, when the window has passed them, and are
+request is released or, in a windowed or chunked group, when no later query sees them, and are
 handed out again without being cleared: nothing reads beyond a request's length.
 The reference's page is one token (crates/infer-protocol/src/config.rs:236-238); the
 partially filled last page is this engine's own.
@@ -85,16 +85,14 @@ class PageGroup:
         return self._np_tables[rid][:len(self.tables[rid])]
 
     def first_needed_page(self, next_pos: int) -> int:
-        """Pages below this index are no longer read by the window once the next query is at ``next_pos``."""
-        if self.need.window is None:
-            return 0
-        return max(0, next_pos - self.need.window + 1) // self.page_size
+        """Pages below this index are no longer read by the window or chunk once the next query is at ``next_pos``."""
+        return self.need.first_position(next_pos) // self.page_size
 
     @property
     def kept_pages(self) -> int:
         """The first pages of a request that are never given back: they hold positions every query may read."""
         keep = getattr(self.need, "keep_first", 0) or 0
-        return pages_for(keep, self.page_size) if self.need.window is not None else 0
+        return pages_for(keep, self.page_size) if self.need.bounded else 0
 
     def droppable(self, next_pos: int) -> range:
         """Indices of the table entries no query at ``next_pos`` or later reads."""
@@ -321,7 +319,7 @@ class CacheManager:
                 if len(t) != want:
                     raise CacheError(f"group {g.index}: request {rid!r} has {len(t)} table entries "
                                      f"for {self._kv_len[rid]} tokens")
-                if g.need.window is None and any(p < 0 for p in t):
+                if not g.need.bounded and any(p < 0 for p in t):
                     raise CacheError(f"group {g.index}: request {rid!r} lost a page")
         if len(self._slot_of) != self.slots.outstanding:
             raise CacheError("slot count does not match live requests")

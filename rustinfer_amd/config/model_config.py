@@ -1198,3 +1198,170 @@ class DebuzenConfig(ModelConfig):
         if self.eos_token_ids:
             d["eos_token_id"] = list(self.eos_token_ids)
         return d
+
+
+# ---------------------------------------------------------------------------
+# Zotonex: attention as the difference of two maps inside chunks, clipped experts whose input is weighted
+# ---------------------------------------------------------------------------
+@dataclass(frozen=True)
+class DifferenceAttentionSpec:
+    """Mixer ``attention``: every head is the difference of two softmax maps (queries and keys of ``dim`` a map,
+    normed) over one set of values (``vdim``); a query sees the keys of its own chunk of ``chunk`` positions
+    (None: all earlier ones); ``diff`` is the constant in the second map's weight; ``kv_from``: the layer whose keys
+    and values this one reads instead of making its own."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    diff: float
+    chunk: Optional[int] = None
+    kv_from: Optional[int] = None
+    kind: str = "attention"
+
+    @staticmethod
+    def from_dict(m: Dict[str, Any], where: str) -> "DifferenceAttentionSpec":
+        mask, kv_from = m.get("mask"), m.get("kv_from")
+        if mask is not None and not isinstance(mask, dict):
+            raise ConfigError(f"{where}: 'mask' must be an object or null")
+        s = DifferenceAttentionSpec(
+            heads=_require(m, "heads", int, where), kv_heads=_require(m, "kv_heads", int, where),
+            dim=_require(m, "dim", int, where), vdim=_require(m, "vdim", int, where),
+            scale=_require(m, "scale", float, where), diff=_require(m, "diff", float, where),
+            chunk=_require(mask, "size", int, where + ".mask") if mask is not None else None,
+            kv_from=_typed(kv_from, "kv_from", int, where) if kv_from is not None else None)
+        if min(s.heads, s.kv_heads, s.dim, s.vdim) <= 0 or s.heads % s.kv_heads:
+            raise ConfigError(f"{where}: heads, kv_heads, dim and vdim must be > 0 and heads a multiple of kv_heads")
+        if s.chunk is not None and s.chunk <= 0:
+            raise ConfigError(f"{where}.mask: size must be > 0")
+        if max(s.dim, s.vdim) > MAX_HEAD_DIM or s.heads // s.kv_heads > 16:
+            raise ConfigError(f"{where}: heads of more than {MAX_HEAD_DIM} features or more than 16 query heads of two "
+                              f"maps a key/value head are beyond the attention kernels")
+        return s
+
+    def to_dict(self) -> Dict[str, Any]:
+        d = {"heads": self.heads, "kv_heads": self.kv_heads, "dim": self.dim, "vdim": self.vdim, "scale": self.scale,
+             "diff": self.diff}
+        if self.chunk is not None:
+            d["mask"] = {"size": self.chunk}
+        if self.kv_from is not None:
+            d["kv_from"] = self.kv_from
+        return d
+
+
+@dataclass(frozen=True)
+class ZotonexExperts:
+    """The feed-forward ``moe``: ``experts`` clipped gated feed-forwards of width ``ff`` (clipped at ``limit``) of
+    which a token uses ``top``, and a gated shared one of width ``shared_ff`` (0: none; clipped at ``shared_limit``)."""
+    ff: int
+    limit: float
+    experts: int
+    top: int
+    shared_ff: int = 0
+    shared_limit: float = 0.0
+
+    @staticmethod
+    def from_dict(mlp: Dict[str, Any], where: str) -> "ZotonexExperts":
+        kind = _require(mlp, "kind", str, where)
+        if kind != "moe":
+            raise ConfigError(f"{where}: unknown feed-forward kind {kind!r} (known: moe)")
+        router, expert, shared = _obj(mlp, "router", where), _obj(mlp, "expert", where), mlp.get("shared")
+        if shared is not None and not isinstance(shared, dict):
+            raise ConfigError(f"{where}: 'shared' must be an object or null")
+        s = ZotonexExperts(
+            _require(expert, "ff", int, where + ".expert"), _require(expert, "limit", float, where + ".expert"),
+            _require(router, "experts", int, where + ".router"), _require(router, "top", int, where + ".router"),
+            _require(shared, "ff", int, where + ".shared") if shared is not None else 0,
+            _require(shared, "limit", float, where + ".shared") if shared is not None else 0.0)
+        if not (0 < s.top <= s.experts) or s.experts > 512:
+            raise ConfigError(f"{where}.router: need 0 < top <= experts <= 512")
+        if s.ff <= 0 or s.shared_ff < 0 or not s.limit > 0 or (s.shared_ff and not s.shared_limit > 0):
+            raise ConfigError(f"{where}: ff and limit must be > 0")
+        return s
+
+    def to_dict(self) -> Dict[str, Any]:
+        d = {"kind": "moe", "expert": {"ff": self.ff, "limit": self.limit}, "router": {"experts": self.experts, "top": self.top}}
+        if self.shared_ff:
+            d["shared"] = {"ff": self.shared_ff, "limit": self.shared_limit}
+        return d
+
+
+ZOTONEX_MIXERS = {"attention": DifferenceAttentionSpec}
+
+
+@dataclass(frozen=True)
+class ZotonexLayer:
+    mixer: Any                                # one of the specs above
+    mlp: Optional[ZotonexExperts] = None      # None: the layer has no feed-forward
+
+    @property
+    def type(self) -> str:
+        return self.mixer.kind
+
+
+@dataclass(frozen=True)
+class ZotonexConfig(ModelConfig):
+    """``{"architecture": "Zotonex", "vocab", "width", "norm": {"eps"}, "embedding": {"scale"}, "logit_scale",
+    "layers": [{"type", "mixer": {...}, "mlp": {...} | null}]}``.  Pre-norm layers; the head has a matrix of its own
+    and its logits are multiplied by ``logit_scale``; no end-of-sequence token of its own."""
+
+    vocab_size: int = 0
+    hidden_size: int = 0
+    norm_eps: float = 1e-6
+    embedding_scale: float = 1.0
+    logit_scale: float = 1.0
+    layers: tuple = ()
+    eos_token_ids: tuple = ()
+    architecture: str = "Zotonex"
+
+    @classmethod
+    def from_dict(cls, d: Dict[str, Any], where: str = "config.json") -> "ZotonexConfig":
+        layers_in = d.get("layers")
+        if not isinstance(layers_in, list) or not layers_in:
+            raise ConfigError(f"{where}: 'layers' must be a non-empty list")
+        layers = []
+        for i, entry in enumerate(layers_in):
+            w = f"{where}.layers[{i}]"
+            if not isinstance(entry, dict):
+                raise ConfigError(f"{w}: must be an object")
+            kind = _require(entry, "type", str, w)
+            if kind not in ZOTONEX_MIXERS:
+                raise ConfigError(f"{w}: unknown mixer type {kind!r} (known: {', '.join(sorted(ZOTONEX_MIXERS))})")
+            mixer = ZOTONEX_MIXERS[kind].from_dict(_obj(entry, "mixer", w), w + ".mixer")
+            mlp = entry.get("mlp")
+            if mlp is not None and not isinstance(mlp, dict):
+                raise ConfigError(f"{w}: 'mlp' must be null or an object")
+            layers.append(ZotonexLayer(mixer, ZotonexExperts.from_dict(mlp, w + ".mlp") if mlp is not None else None))
+        for i, layer in enumerate(layers):
+            j = layer.mixer.kv_from
+            if j is None:
+                continue
+            w = f"{where}.layers[{i}].mixer"
+            if not (0 <= j < i) or layers[j].mixer.kv_from is not None:
+                raise ConfigError(f"{w}: kv_from must name an earlier layer that has keys and values of its own")
+            a, b = layer.mixer, layers[j].mixer
+            if (a.kv_heads, a.dim, a.vdim) != (b.kv_heads, b.dim, b.vdim):
+                raise ConfigError(f"{w}: kv_heads, dim and vdim must equal those of layer {j}, whose keys and values it reads")
+        eos = d.get("eos_token_id")
+        eos_ids = () if eos is None else tuple(_typed(e, "eos_token_id", int, where) for e in (eos if isinstance(eos, list) else [eos]))
+        emb = d.get("embedding")
+        if emb is not None and not isinstance(emb, dict):
+            raise ConfigError(f"{where}: 'embedding' must be an object")
+        cfg = cls(vocab_size=_require(d, "vocab", int, where), hidden_size=_require(d, "width", int, where),
+                  norm_eps=_require(_obj(d, "norm", where), "eps", float, where + ".norm"),
+                  embedding_scale=_typed(emb.get("scale", 1.0), "scale", float, where + ".embedding") if emb else 1.0,
+                  logit_scale=_typed(d.get("logit_scale", 1.0), "logit_scale", float, where),
+                  layers=tuple(layers), eos_token_ids=eos_ids)
+        if cfg.vocab_size <= 0 or cfg.hidden_size <= 0 or not cfg.norm_eps > 0:
+            raise ConfigError(f"{where}: vocab and width must be > 0, norm.eps > 0")
+        return cfg
+
+    def to_dict(self) -> Dict[str, Any]:
+        d: Dict[str, Any] = {
+            "architecture": self.architecture, "vocab": self.vocab_size, "width": self.hidden_size,
+            "norm": {"eps": self.norm_eps}, "embedding": {"scale": self.embedding_scale}, "logit_scale": self.logit_scale,
+            "layers": [{"type": l.type, "mixer": l.mixer.to_dict(), "mlp": None if l.mlp is None else l.mlp.to_dict()}
+                       for l in self.layers]}
+        if self.eos_token_ids:
+            d["eos_token_id"] = list(self.eos_token_ids)
+        return d

@@ -4,7 +4,8 @@
 //   head_norm_kv_write   queries and keys divided by their root mean square over the head, times a
 //                        weight of the head's size shared by all heads, the query times a
 //                        temperature that grows with the logarithm of its position; the query in
-//                        place, the normed key and the value into the token's page;
+//                        place, the normed key and the value into the token's page (a head may hold
+//                        several queries or keys side by side, each normed on its own);
 //   latent_kv_write      attention through one latent vector a token: the first R features of the
 //                        down projection are normed (c), the last r are one rotated key part for all
 //                        heads; the page takes the key [c, rotated part] and the value c; the
@@ -29,22 +30,23 @@ __global__ __launch_bounds__(256) void head_norm_kv_write_kernel(
         T* __restrict__ q, int q_stride, const T* __restrict__ k, int k_stride, const T* __restrict__ v, int v_stride,
         int H, int Hkv, int dk, int dv, const float* __restrict__ qw, const float* __restrict__ kw, int do_norm, float eps,
         float temp_coef, int temp_every, const int* __restrict__ positions, const int* __restrict__ row_of_token,
-        T* __restrict__ kc, T* __restrict__ vc, const int* __restrict__ table, int max_blocks, int page, int write_kv) {
+        T* __restrict__ kc, T* __restrict__ vc, const int* __restrict__ table, int max_blocks, int page, int write_kv, int maps) {
     const int t = blockIdx.x;
     const int b = row_of_token[t];
     if (b < 0) return;                       // padding token
     const int pos = positions[t];
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int Hq = H * maps, Hk = Hkv * maps;          // what is normed: every map of every head
     int blk = -1;
     if (write_kv) blk = table[(size_t)b * max_blocks + pos / page];
     const int slot = pos % page;
     const float temp = temp_every > 0 ? 1.f + temp_coef * logf((float)((pos + 1) / temp_every) + 1.f) : 1.f;
-    const int units = H + (blk >= 0 ? Hkv : 0);
+    const int units = Hq + (blk >= 0 ? Hk : 0);
     for (int u = blockIdx.y * 4 + wave; u < units; u += 4 * gridDim.y) {
-        const bool is_q = u < H;
-        const int g = u - H;
+        const bool is_q = u < Hq;
+        const int g = is_q ? 0 : u - Hq;
         const T* src = is_q ? q + (size_t)t * q_stride + u * dk : k + (size_t)t * k_stride + g * dk;
-        T* dst = is_q ? q + (size_t)t * q_stride + u * dk : kc + (((size_t)blk * Hkv + g) * page + slot) * dk;
+        T* dst = is_q ? q + (size_t)t * q_stride + u * dk : kc + (((size_t)blk * Hkv + g / maps) * page + slot) * (maps * dk) + g % maps * dk;
         const float* w = is_q ? qw : kw;
         float f = is_q ? temp : 1.f;
         if (do_norm) {
@@ -226,25 +228,27 @@ __global__ __launch_bounds__(256) void head_linear_few_kernel(
 // (write_kv; a layer that reads another layer's cache has none).  qw, kw: 32-bit weights of dk
 // entries or null; do_norm 0: no division by the root mean square (weights and temperature only).
 // temp_every > 0: the query at position p is multiplied by 1 + temp_coef ln(floor((p + 1) / temp_every) + 1).
+// maps: queries a query head and keys a key head hold, side by side (q [T][>= H maps dk], k [T][>= Hkv maps dk]);
+// each is normed on its own with the same weight, and the cached key row has maps dk features.
 extern "C" int ri_head_norm_kv_write(
         void* q, int q_stride, const void* k, int k_stride, const void* v, int v_stride, int dtype, int T,
         int H, int Hkv, int dk, int dv, const float* qw, const float* kw, int do_norm, float eps,
         float temp_coef, int temp_every, const int* positions, const int* row_of_token,
-        void* kc, void* vc, int num_pages, const int* table, int max_blocks, int page, int write_kv, hipStream_t stream) {
-    RI_REQUIRE(T >= 0 && H > 0 && Hkv > 0 && dk > 0 && dv > 0 && page > 0, "ri_head_norm_kv_write: bad sizes");
-    RI_REQUIRE(q_stride >= H * dk, "ri_head_norm_kv_write: query row stride %d too small", q_stride);
+        void* kc, void* vc, int num_pages, const int* table, int max_blocks, int page, int write_kv, int maps, hipStream_t stream) {
+    RI_REQUIRE(T >= 0 && H > 0 && Hkv > 0 && dk > 0 && dv > 0 && page > 0 && maps > 0, "ri_head_norm_kv_write: bad sizes");
+    RI_REQUIRE(q_stride >= H * maps * dk, "ri_head_norm_kv_write: query row stride %d too small", q_stride);
     RI_REQUIRE(!do_norm || eps > 0.f, "ri_head_norm_kv_write: eps must be > 0");
-    if (write_kv) RI_REQUIRE(k && v && kc && vc && table && max_blocks > 0 && num_pages > 0 && k_stride >= Hkv * dk && v_stride >= Hkv * dv,
+    if (write_kv) RI_REQUIRE(k && v && kc && vc && table && max_blocks > 0 && num_pages > 0 && k_stride >= Hkv * maps * dk && v_stride >= Hkv * dv,
                              "ri_head_norm_kv_write: no keys, values or cache given, or their row strides too small");
     if (T == 0) return 0;
     RI_REQUIRE(q && positions && row_of_token, "ri_head_norm_kv_write: null pointer");
     // a step of few tokens: a block for every four heads, so that no wave walks a chain of heads
-    const int by = T <= 256 ? min((H + Hkv + 3) / 4, 64) : 1;
+    const int by = T <= 256 ? min(((H + Hkv) * maps + 3) / 4, 64) : 1;
     const dim3 grid(T, by);
     if (dtype == RI_F32)
-        head_norm_kv_write_kernel<float><<<grid, 256, 0, stream>>>((float*)q, q_stride, (const float*)k, k_stride, (const float*)v, v_stride, H, Hkv, dk, dv, qw, kw, do_norm, eps, temp_coef, temp_every, positions, row_of_token, (float*)kc, (float*)vc, table, max_blocks, page, write_kv);
+        head_norm_kv_write_kernel<float><<<grid, 256, 0, stream>>>((float*)q, q_stride, (const float*)k, k_stride, (const float*)v, v_stride, H, Hkv, dk, dv, qw, kw, do_norm, eps, temp_coef, temp_every, positions, row_of_token, (float*)kc, (float*)vc, table, max_blocks, page, write_kv, maps);
     else if (dtype == RI_BF16)
-        head_norm_kv_write_kernel<bf16_t><<<grid, 256, 0, stream>>>((bf16_t*)q, q_stride, (const bf16_t*)k, k_stride, (const bf16_t*)v, v_stride, H, Hkv, dk, dv, qw, kw, do_norm, eps, temp_coef, temp_every, positions, row_of_token, (bf16_t*)kc, (bf16_t*)vc, table, max_blocks, page, write_kv);
+        head_norm_kv_write_kernel<bf16_t><<<grid, 256, 0, stream>>>((bf16_t*)q, q_stride, (const bf16_t*)k, k_stride, (const bf16_t*)v, v_stride, H, Hkv, dk, dv, qw, kw, do_norm, eps, temp_coef, temp_every, positions, row_of_token, (bf16_t*)kc, (bf16_t*)vc, table, max_blocks, page, write_kv, maps);
     else
         return ri_fail("ri_head_norm_kv_write: unknown dtype %d", dtype);
     RI_LAUNCHED("ri_head_norm_kv_write");

@@ -8,6 +8,13 @@
 // Query token t of request row b at position p, head h (key/value head g = h / (H / Hkv)):
 //   keys j in [max(0, p + 1 - window), min(kv_len_b, p + 1)),  s_j = (q . K_j) * scale,
 //   out = turn(-p) sum_j softmax(s)_j V_j.
+// Instead of a window, or beside it, positions may be cut into chunks of `chunk` counted from the
+// request's first position: a query sees keys of its own chunk only (j >= p - p mod chunk).
+// maps = 2: a query head holds two queries and a key head two keys of dk features each, side by side
+// (first map, second map), over one set of values; H counts query heads, and in the kernels every map
+// of a head is a head of its own (2 H of them) whose keys are its map's half of the key row.  A head's output is
+// the difference of its two maps' outputs, o = a - lam b, divided by its root mean square over the
+// head's dv values (diff_eps inside the root) and multiplied by diff_gain; a and b stay 32-bit.
 // Storage is 32-bit or bfloat16; scores, weights, sums and the turns are 32-bit.
 // Cache layout: keys [pages][Hkv][page][dk], values [pages][Hkv][dv][page] (positions of a
 // feature contiguous).
@@ -119,6 +126,32 @@ __global__ __launch_bounds__(256) void rotate_kv_write_kernel(
     }
 }
 
+// The first key a query at position p sees (kept first positions aside).
+__device__ __forceinline__ int aw_first_key(int p, int window, int chunk) {
+    int lo = window > 0 ? max(0, p + 1 - window) : 0;
+    if (chunk > 0) lo = max(lo, p - p % chunk);
+    return lo;
+}
+
+// How the outputs of a head's two maps become one (maps = 2).
+struct DiffHow { float lam, gain, eps; };
+
+// A wave writes a head's output from its two maps' outputs, NC values of each a lane (feature lane + 64 c).
+template <typename T, int NC>
+__device__ __forceinline__ void aw_write_difference(T* __restrict__ o, const float (&a)[NC], const float (&b)[NC], int dv, int lane, DiffHow how) {
+    float y[NC], ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < NC; ++c) {
+        y[c] = lane + 64 * c < dv ? a[c] - how.lam * b[c] : 0.f;
+        ss = fmaf(y[c], y[c], ss);
+    }
+    ss = wave_sum(ss);
+    const float f = how.gain / sqrtf(ss / (float)dv + how.eps);
+#pragma unroll
+    for (int c = 0; c < NC; ++c)
+        if (lane + 64 * c < dv) st_f32(o + lane + 64 * c, y[c] * f);
+}
+
 // One row's scores against the keys of a block, one key a lane: the block's maximum, the weights
 // relative to it and their sum.  m_b = -inf (l_b = 0) if the row sees no key of the block.
 __device__ __forceinline__ float aw_block_scores(float dot, bool mine, float scale, float& m_b, float& l_b) {
@@ -182,13 +215,14 @@ __global__ __launch_bounds__(256) void attn_window_kernel(
         const int* __restrict__ cu_q, const int* __restrict__ q_start, const int* __restrict__ kv_lens,
         int num_rows, int H, int Hkv, int dk, int dv, int page, float scale, int window, int TQ, int NK,
         const float* __restrict__ vcos, const float* __restrict__ vsin, int v_interleaved, const float* __restrict__ sink,
-        int keep, const float* __restrict__ sig_bias) {
+        int keep, const float* __restrict__ sig_bias, int chunk, int maps, DiffHow diff) {
     extern __shared__ __align__(16) float lds[];
-    const int dkp = (dk + 3) & ~3, ks_stride = dkp + 4, vs_stride = dv + 1;
+    // (maps = 2: map m of a key lies at m * dkp of its row)
+    const int dkp = (dk + 3) & ~3, dkr = maps * dk, ks_stride = maps * dkp + 4, vs_stride = dv + 1;
     float* Qs = lds;                                   // [AW_ROWS][dkp]
     float* Ps = Qs + AW_ROWS * dkp;                    // [AW_ROWS][NK]
     int* koff = reinterpret_cast<int*>(Ps + AW_ROWS * NK);      // [64] key slot in the cache, -1: none
-    float* Ks = reinterpret_cast<float*>(koff + 64);   // [NK][dkp + 4]
+    float* Ks = reinterpret_cast<float*>(koff + 64);   // [NK][maps dkp + 4]
     float* Vs = Ks + NK * ks_stride;                   // [NK][dv + 1]
     float* Os = Ks;                                    // [AW_ROWS][dv], after the last block of keys
 
@@ -210,7 +244,7 @@ __global__ __launch_bounds__(256) void attn_window_kernel(
     const int p0 = q_start[b] + (t0 - cu_q[b]);        // position of the tile's first token
     const int kv_len = kv_lens[b];
     const int last_visible = min(kv_len, p0 + nt);
-    const int first_key = window > 0 ? max(0, p0 + 1 - window) : 0;
+    const int first_key = aw_first_key(p0, window, chunk);
 
     for (int e = tid; e < AW_ROWS * dkp; e += 256) {
         const int r = e / dkp, dd = e - r * dkp;
@@ -227,7 +261,7 @@ __global__ __launch_bounds__(256) void attn_window_kernel(
         for (int c = 0; c < NC; ++c) acc[i][c] = 0.f;
         const int r = wave + 4 * i, p = p0 + r / G;
         row_hi[i] = r < R ? min(kv_len, p + 1) : 0;
-        row_lo[i] = window > 0 ? max(0, p + 1 - window) : 0;
+        row_lo[i] = aw_first_key(p, window, chunk);
     }
 
     // keep > 0: the first `keep` positions stay in sight behind the window: their blocks of keys first
@@ -247,21 +281,21 @@ __global__ __launch_bounds__(256) void attn_window_kernel(
         __syncthreads();
         constexpr int VL = 16 / sizeof(T);              // elements of a 16-byte load
         if (dk % VL == 0) {                            // keys: 16 bytes a thread and load
-            const int pieces = dk / VL;
+            const int pieces = dkr / VL;               // (dkp = dk here: the maps lie side by side)
             for (int e = tid; e < NK * pieces; e += 256) {
                 const int jj = e / pieces, pc = e - jj * pieces, off = koff[jj];
                 float f[VL];
 #pragma unroll
                 for (int u = 0; u < VL; ++u) f[u] = 0.f;
-                if (off >= 0) ld_vec16(kc + (size_t)off * dk + pc * VL, f);
+                if (off >= 0) ld_vec16(kc + (size_t)off * dkr + pc * VL, f);
 #pragma unroll
                 for (int u = 0; u < VL; u += 4)
                     *reinterpret_cast<float4*>(Ks + jj * ks_stride + pc * VL + u) = make_float4(f[u], f[u + 1], f[u + 2], f[u + 3]);
             }
         } else {
-            for (int e = tid; e < NK * dkp; e += 256) {
-                const int jj = e / dkp, dd = e - jj * dkp, off = koff[jj];
-                Ks[jj * ks_stride + dd] = (off >= 0 && dd < dk) ? ld_f32(kc + (size_t)off * dk + dd) : 0.f;
+            for (int e = tid; e < NK * maps * dkp; e += 256) {
+                const int jj = e / (maps * dkp), at = e - jj * maps * dkp, m_ = at / dkp, dd = at - m_ * dkp, off = koff[jj];
+                Ks[jj * ks_stride + at] = (off >= 0 && dd < dk) ? ld_f32(kc + (size_t)off * dkr + m_ * dk + dd) : 0.f;
             }
         }
         if (page % VL == 0) {
@@ -304,7 +338,8 @@ __global__ __launch_bounds__(256) void attn_window_kernel(
             // rows of this batch that exist for this wave (a step of single tokens has G rows a tile)
             const int nrb = min(4, (R - wave + 3) / 4 - 4 * bi);
             float s[4] = {0.f, 0.f, 0.f, 0.f};
-            const float* kr = Ks + (lane < NK ? lane : 0) * ks_stride;
+            // two maps: an even number of heads a group, so a wave's rows (wave + 4 i) are all of one map
+            const float* kr = Ks + (lane < NK ? lane : 0) * ks_stride + (maps == 2 ? (wave & 1) * dkp : 0);
 #pragma unroll 2
             for (int dd = 0; dd < dkp; dd += 4) {
                 const float4 k4 = *reinterpret_cast<const float4*>(kr + dd);
@@ -359,6 +394,33 @@ __global__ __launch_bounds__(256) void attn_window_kernel(
 #pragma unroll
         for (int i = 0; i < 8; ++i) aw_merge<NC>(m[i], l[i], acc[i], m_b[i], l_b[i], acc_b[i]);
     }
+    if (maps == 2) {
+        // the two maps of a head lie in neighbouring rows, in different waves: through LDS
+        __syncthreads();                               // the last keys and values have been used
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+            const int r = wave + 4 * i;
+            if (r >= R) continue;
+            const float fin = sig_bias ? 1.f : aw_final_factor(m[i], l[i], sink, g * G + r % G);
+#pragma unroll
+            for (int c = 0; c < NC; ++c) {
+                const int d = lane + 64 * c;
+                if (d < dv) Os[r * dv + d] = acc[i][c] * fin;
+            }
+        }
+        __syncthreads();
+        for (int r = 2 * wave; r < R; r += 8) {
+            float a[NC], bb[NC];
+#pragma unroll
+            for (int c = 0; c < NC; ++c) {
+                const int d = lane + 64 * c;
+                a[c] = d < dv ? Os[r * dv + d] : 0.f;
+                bb[c] = d < dv ? Os[(r + 1) * dv + d] : 0.f;
+            }
+            aw_write_difference<T, NC>(out + (size_t)(t0 + r / G) * out_stride + (g * G + r % G) / 2 * dv, a, bb, dv, lane, diff);
+        }
+        return;
+    }
     if (vcos == nullptr) {
 #pragma unroll
         for (int i = 0; i < 8; ++i) {
@@ -411,55 +473,74 @@ __device__ __forceinline__ int aw_keep_used(int keep, int NK, int first_key, int
 
 // Steps of single tokens: merge the partial results of a row's blocks of keys in ascending order
 // (the order and the arithmetic of the loop in attn_window_kernel), divide, turn back, write.
-// One wave a (token, head).
-template <typename T, int NC>
+// One wave a (token, head); with two maps a head it merges both and writes their difference.
+template <typename T, int NC, int MAPS>
 __global__ __launch_bounds__(64) void attn_window_combine_kernel(
         const float* __restrict__ part_ml, const float* __restrict__ part_o, T* __restrict__ out, int out_stride,
         const int* __restrict__ cu_q, const int* __restrict__ q_start, const int* __restrict__ kv_lens,
         int H, int dv, int window, int NK, int slots,
         const float* __restrict__ vcos, const float* __restrict__ vsin, int v_interleaved, const float* __restrict__ sink,
-        int keep, int sigmoid_weights) {
+        int keep, int sigmoid_weights, int chunk, DiffHow diff) {
     __shared__ float Os[256];
-    const int b = blockIdx.y, h = blockIdx.x, lane = threadIdx.x;
+    const int b = blockIdx.y, ho = blockIdx.x, lane = threadIdx.x;
     const int t = cu_q[b];
     if (cu_q[b + 1] - t <= 0) return;                  // a row without a token
     const int p = q_start[b];
     const int visible = min(kv_lens[b], p + 1);
-    const int first_key = window > 0 ? max(0, p + 1 - window) : 0;
+    const int first_key = aw_first_key(p, window, chunk);
     // the first slots belong to the blocks of the kept positions (those that lie before the window's first block)
     const int keep_slots = (keep + NK - 1) / NK, keep_used = aw_keep_used(keep, NK, first_key, visible);
     const int n = keep_slots + (visible + NK - 1) / NK - first_key / NK;
-    float m = -INFINITY, l = 0.f, acc[NC];
+    float m[MAPS], l[MAPS], acc[MAPS][NC];
 #pragma unroll
-    for (int c = 0; c < NC; ++c) acc[c] = 0.f;
+    for (int k = 0; k < MAPS; ++k) {
+        m[k] = -INFINITY;
+        l[k] = 0.f;
+#pragma unroll
+        for (int c = 0; c < NC; ++c) acc[k][c] = 0.f;
+    }
     // eight blocks' partial results are asked for at once, then merged one after the other in the
     // order of the blocks: the loads of a block do not wait for the merge of the one before
-    constexpr int AHEAD = 8;
+    constexpr int AHEAD = 8 / MAPS;
     const int count = min(n, slots);
     for (int s0 = 0; s0 < count; s0 += AHEAD) {
-        float acc_b[AHEAD][NC], m_b[AHEAD], l_b[AHEAD];
+        float acc_b[MAPS][AHEAD][NC], m_b[MAPS][AHEAD], l_b[MAPS][AHEAD];
 #pragma unroll
-        for (int i = 0; i < AHEAD; ++i) {
-            const bool on = s0 + i < count && (s0 + i >= keep_slots || s0 + i < keep_used);
-            const size_t at = ((size_t)t * H + h) * slots + (on ? s0 + i : 0);
-            m_b[i] = on ? part_ml[at * 2] : -INFINITY;
-            l_b[i] = on ? part_ml[at * 2 + 1] : 0.f;
+        for (int k = 0; k < MAPS; ++k)
 #pragma unroll
-            for (int c = 0; c < NC; ++c) {
-                const int d = lane + 64 * c;
-                acc_b[i][c] = (on && d < dv) ? part_o[at * dv + d] : 0.f;
+            for (int i = 0; i < AHEAD; ++i) {
+                const bool on = s0 + i < count && (s0 + i >= keep_slots || s0 + i < keep_used);
+                const size_t at = ((size_t)t * H + ho * MAPS + k) * slots + (on ? s0 + i : 0);
+                m_b[k][i] = on ? part_ml[at * 2] : -INFINITY;
+                l_b[k][i] = on ? part_ml[at * 2 + 1] : 0.f;
+#pragma unroll
+                for (int c = 0; c < NC; ++c) {
+                    const int d = lane + 64 * c;
+                    acc_b[k][i][c] = (on && d < dv) ? part_o[at * dv + d] : 0.f;
+                }
             }
-        }
 #pragma unroll
-        for (int i = 0; i < AHEAD; ++i)
-            if (s0 + i < count) aw_merge<NC>(m, l, acc, m_b[i], l_b[i], acc_b[i]);        // (a slot that is off has m_b = -inf)
+        for (int k = 0; k < MAPS; ++k)
+#pragma unroll
+            for (int i = 0; i < AHEAD; ++i)
+                if (s0 + i < count) aw_merge<NC>(m[k], l[k], acc[k], m_b[k][i], l_b[k][i], acc_b[k][i]);        // (a slot that is off has m_b = -inf)
     }
-    T* o = out + (size_t)t * out_stride + h * dv;
+    T* o = out + (size_t)t * out_stride + ho * dv;
+    if constexpr (MAPS == 2) {
+#pragma unroll
+        for (int k = 0; k < 2; ++k) {
+            const float fin = sigmoid_weights ? 1.f : aw_final_factor(m[k], l[k], sink, ho * 2 + k);
+#pragma unroll
+            for (int c = 0; c < NC; ++c) acc[k][c] *= fin;
+        }
+        aw_write_difference<T, NC>(o, acc[0], acc[1], dv, lane, diff);
+        return;
+    }
 #pragma unroll
     for (int c = 0; c < NC; ++c) {
         const int d = lane + 64 * c;
         if (d < dv) {
-            const float y = sigmoid_weights ? acc[c] : sink ? acc[c] * aw_final_factor(m, l, sink, h) : (l > 0.f ? acc[c] / l : 0.f);
+            const float y = sigmoid_weights ? acc[0][c] : sink ? acc[0][c] * aw_final_factor(m[0], l[0], sink, ho) : (l[0] > 0.f ? acc[0][c] / l[0] : 0.f);
             if (vcos == nullptr) st_f32(o + d, y);
             else Os[d] = y;
         }
@@ -484,12 +565,13 @@ __global__ __launch_bounds__(64) void attn_window_combine_kernel(
 // same arithmetic, term for term, as a block of keys in attn_window_kernel.
 constexpr int AD_KEYS = 64;
 
-template <typename T, int NC>
+template <typename T, int NC, int MAPS>
 __global__ __launch_bounds__(256) void attn_window_decode_kernel(
         const T* __restrict__ q, int q_stride, const T* __restrict__ kc, const T* __restrict__ vc,
         const int* __restrict__ table, int max_blocks, const int* __restrict__ cu_q, const int* __restrict__ q_start,
         const int* __restrict__ kv_lens, int H, int Hkv, int dk, int dv, int page, float scale, int window, int slots,
-        float* __restrict__ part_ml, float* __restrict__ part_o, int heads_a_wave, int keep, const float* __restrict__ sig_bias) {
+        float* __restrict__ part_ml, float* __restrict__ part_o, int heads_a_wave, int keep, const float* __restrict__ sig_bias,
+        int chunk) {
     extern __shared__ __align__(16) float lds[];       // [4 waves][G][64] weights
     // many query heads a key/value head (one shared latent, say): the heads are dealt to several
     // blocks in stretches of heads_a_wave, each reading the block of keys for its own heads
@@ -501,7 +583,7 @@ __global__ __launch_bounds__(256) void attn_window_decode_kernel(
     if (cu_q[b + 1] - t <= 0) return;                  // a row without a token
     const int p = q_start[b];
     const int visible = min(kv_lens[b], p + 1);
-    const int j0 = window > 0 ? max(0, p + 1 - window) : 0;
+    const int j0 = aw_first_key(p, window, chunk);
     const int slot = (int)blockIdx.x * 4 + wave;
     const int keep_slots = (keep + AD_KEYS - 1) / AD_KEYS;
     if (slot < keep_slots && slot >= aw_keep_used(keep, AD_KEYS, j0, visible)) return;
@@ -519,7 +601,7 @@ __global__ __launch_bounds__(256) void attn_window_decode_kernel(
         own_pid = pid;
         if (pid >= 0) off = ((long long)pid * Hkv + g) * page + j % page;
     }
-    const T* kr = off >= 0 ? kc + (size_t)off * dk : nullptr;
+    const T* kr = off >= 0 ? kc + (size_t)off * (MAPS * dk) : nullptr;
     const T* qrow = q + (size_t)t * q_stride + (size_t)g * G * dk;
     const size_t at0 = ((size_t)t * H + (size_t)g * G) * slots + slot;      // + head * slots
     const bool kvec = dk % VL == 0;
@@ -527,25 +609,30 @@ __global__ __launch_bounds__(256) void attn_window_decode_kernel(
         float s[4] = {0.f, 0.f, 0.f, 0.f};
         if (kvec) {
             for (int dd = 0; dd < dk; dd += VL) {
-                float kf[VL];
+                float kf[MAPS][VL];                    // (two maps: h0 is even, so head h0 + rb is of map rb % 2)
 #pragma unroll
-                for (int u = 0; u < VL; ++u) kf[u] = 0.f;
-                if (kr) ld_vec16(kr + dd, kf);
+                for (int k = 0; k < MAPS; ++k) {
+#pragma unroll
+                    for (int u = 0; u < VL; ++u) kf[k][u] = 0.f;
+                    if (kr) ld_vec16(kr + k * dk + dd, kf[k]);
+                }
 #pragma unroll
                 for (int rb = 0; rb < 4; ++rb) {
                     if (h0 + rb >= h_hi) break;
                     float qf[VL];
                     ld_vec16(qrow + (size_t)(h0 + rb) * dk + dd, qf);
 #pragma unroll
-                    for (int u = 0; u < VL; ++u) s[rb] = fmaf(qf[u], kf[u], s[rb]);
+                    for (int u = 0; u < VL; ++u) s[rb] = fmaf(qf[u], kf[rb % MAPS][u], s[rb]);
                 }
             }
         } else {
             for (int dd = 0; dd < dk; ++dd) {
-                const float kf = kr ? ld_f32(kr + dd) : 0.f;
+                float kf[MAPS];
+#pragma unroll
+                for (int k = 0; k < MAPS; ++k) kf[k] = kr ? ld_f32(kr + k * dk + dd) : 0.f;
 #pragma unroll
                 for (int rb = 0; rb < 4; ++rb)
-                    if (h0 + rb < h_hi) s[rb] = fmaf(ld_f32(qrow + (size_t)(h0 + rb) * dk + dd), kf, s[rb]);
+                    if (h0 + rb < h_hi) s[rb] = fmaf(ld_f32(qrow + (size_t)(h0 + rb) * dk + dd), kf[rb % MAPS], s[rb]);
             }
         }
 #pragma unroll
@@ -636,36 +723,42 @@ __global__ __launch_bounds__(256) void attn_window_decode_kernel(
     }
 }
 
-int aw_keys_a_block(int dk, int dv);
-
-size_t aw_lds_bytes(int dk, int dv, int NK) {
+size_t aw_lds_bytes(int dk, int dv, int NK, int maps) {
     const int dkp = (dk + 3) & ~3;
-    const size_t kv = (size_t)NK * (dkp + 4) + (size_t)NK * (dv + 1);
+    const size_t kv = (size_t)NK * (maps * dkp + 4) + (size_t)NK * (dv + 1);
     const size_t os = (size_t)AW_ROWS * dv;
     return sizeof(float) * ((size_t)AW_ROWS * dkp + (size_t)AW_ROWS * NK + 64 + (kv > os ? kv : os));
 }
 
 constexpr size_t AW_LDS_MOST = 150 * 1024;
 
-int aw_keys_a_block(int dk, int dv) {
+int aw_keys_a_block(int dk, int dv, int maps) {
     int NK = 64;
-    while (NK > 16 && aw_lds_bytes(dk, dv, NK) > AW_LDS_MOST) NK >>= 1;
+    while (NK > 16 && aw_lds_bytes(dk, dv, NK, maps) > AW_LDS_MOST) NK >>= 1;
     return NK;
 }
 
 // blocks of keys the window of a single token can touch when no request is longer than max_kv_len
-int aw_slots(int dk, int dv, int window, int max_kv_len, int keep) {
+int aw_slots(int window, int chunk, int max_kv_len, int keep) {
     const int NK = AD_KEYS;
-    const int span = window > 0 ? min(window, max_kv_len) : max_kv_len;
-    // a window may begin inside a block: one more; the blocks of the kept positions come first
-    return (span + NK - 1) / NK + (window > 0 ? 1 : 0) + (window > 0 ? (keep + NK - 1) / NK : 0);
+    int span = max_kv_len;
+    if (window > 0) span = min(window, span);
+    if (chunk > 0) span = min(chunk, span);
+    const bool bounded = window > 0 || chunk > 0;
+    // a window or a chunk may begin inside a block: one more; the blocks of the kept positions come first
+    return (span + NK - 1) / NK + (bounded ? 1 : 0) + (bounded ? (keep + NK - 1) / NK : 0);
+}
+
+// H query heads of `maps` maps each on Hkv key/value heads
+bool aw_sizes_ok(int H, int Hkv, int dk, int dv, int maps) {
+    return H > 0 && Hkv > 0 && H % Hkv == 0 && (maps == 1 || maps == 2) && H / Hkv * maps <= AW_ROWS && dk > 0 && dk <= 256
+        && dv > 0 && dv <= 256 && aw_lds_bytes(dk, dv, 16, maps) <= AW_LDS_MOST;
 }
 
 }  // namespace
 
-extern "C" int ri_attention_window_supported(int H, int Hkv, int dk, int dv) {
-    return H > 0 && Hkv > 0 && H % Hkv == 0 && H / Hkv <= AW_ROWS && dk > 0 && dk <= 256 && dv > 0 && dv <= 256
-        && aw_lds_bytes(dk, dv, 16) <= AW_LDS_MOST;
+extern "C" int ri_attention_window_supported(int H, int Hkv, int dk, int dv, int maps) {
+    return aw_sizes_ok(H, Hkv, dk, dv, maps);
 }
 
 extern "C" int ri_rotate_kv_write(
@@ -698,10 +791,11 @@ template <typename T>
 int aw_launch(const T* q, int q_stride, T* out, int out_stride, const T* kc, const T* vc, const int* table, int max_blocks,
               const int* cu_q, const int* q_start, const int* kv_lens, int num_rows, int Tn, int H, int Hkv, int dk, int dv,
               int page, float scale, int window, const float* vcos, const float* vsin, int v_interleaved,
-              int slots, float* workspace, const float* sink, int keep, const float* sig_bias, hipStream_t stream) {
-    const int G = H / Hkv, TQ = AW_ROWS / G;
-    const int NK = aw_keys_a_block(dk, dv);
-    const size_t lds = aw_lds_bytes(dk, dv, NK);
+              int slots, float* workspace, const float* sink, int keep, const float* sig_bias,
+              int chunk, int maps, DiffHow diff, hipStream_t stream) {
+    const int G = H / Hkv, TQ = AW_ROWS / G;           // (H: the maps of all heads)
+    const int NK = aw_keys_a_block(dk, dv, maps);
+    const size_t lds = aw_lds_bytes(dk, dv, NK, maps);
     const int NC = (dv + 63) / 64;
     auto kernel = NC == 1 ? attn_window_kernel<T, 1> : NC == 2 ? attn_window_kernel<T, 2> : NC == 3 ? attn_window_kernel<T, 3> : attn_window_kernel<T, 4>;
     if (lds > 64 * 1024) {
@@ -717,8 +811,9 @@ int aw_launch(const T* q, int q_stride, T* out, int out_stride, const T* kc, con
         // every row has at most one token: a tile a row, a block a block of keys, then the merge
         float* part_ml = workspace;
         float* part_o = workspace + (size_t)Tn * H * slots * 2;
-        auto part = NC == 1 ? attn_window_decode_kernel<T, 1> : NC == 2 ? attn_window_decode_kernel<T, 2>
-                  : NC == 3 ? attn_window_decode_kernel<T, 3> : attn_window_decode_kernel<T, 4>;
+#define RI_AW_FORM(K) (maps == 2 ? (NC == 1 ? K<T, 1, 2> : NC == 2 ? K<T, 2, 2> : NC == 3 ? K<T, 3, 2> : K<T, 4, 2>) \
+                                 : (NC == 1 ? K<T, 1, 1> : NC == 2 ? K<T, 2, 1> : NC == 3 ? K<T, 3, 1> : K<T, 4, 1>))
+        auto part = RI_AW_FORM(attn_window_decode_kernel);
         // beyond eight heads a key/value head, four heads a wave (one pass over the block of keys): a step
         // of few rows then has waves enough to hide the loads of one another (32 heads on one latent, 8 rows
         // of 2,048 keys: 258 us with all heads in one wave, 78 with eight, 47 with four, 74 with two)
@@ -731,26 +826,26 @@ int aw_launch(const T* q, int q_stride, T* out, int out_stride, const T* kc, con
         RI_REQUIRE((long)Hkv * stretches <= 65535, "ri_attention_window: too many heads for the grid");
         part<<<dim3((slots + 3) / 4, Hkv * stretches, num_rows), 256, sizeof(float) * 4 * G * AD_KEYS, stream>>>(
             q, q_stride, kc, vc, table, max_blocks, cu_q, q_start, kv_lens, H, Hkv, dk, dv, page, scale, window, slots, part_ml, part_o,
-            heads_a_wave, keep, sig_bias);
-        auto combine = NC == 1 ? attn_window_combine_kernel<T, 1> : NC == 2 ? attn_window_combine_kernel<T, 2>
-                     : NC == 3 ? attn_window_combine_kernel<T, 3> : attn_window_combine_kernel<T, 4>;
-        combine<<<dim3(H, num_rows), 64, 0, stream>>>(part_ml, part_o, out, out_stride, cu_q, q_start, kv_lens, H, dv, window, AD_KEYS, slots,
-                                                      vcos, vsin, v_interleaved, sink, keep, sig_bias != nullptr);
+            heads_a_wave, keep, sig_bias, chunk);
+        auto combine = RI_AW_FORM(attn_window_combine_kernel);
+#undef RI_AW_FORM
+        combine<<<dim3(H / maps, num_rows), 64, 0, stream>>>(part_ml, part_o, out, out_stride, cu_q, q_start, kv_lens, H, dv, window, AD_KEYS, slots,
+                                                             vcos, vsin, v_interleaved, sink, keep, sig_bias != nullptr, chunk, diff);
         return 0;
     }
     const int tiles = (Tn + TQ - 1) / TQ + num_rows;   // at most: every request may end in a short tile
     kernel<<<dim3(tiles, Hkv), 256, lds, stream>>>(q, q_stride, out, out_stride, kc, vc, table, max_blocks, cu_q, q_start, kv_lens,
                                                    num_rows, H, Hkv, dk, dv, page, scale, window, TQ, NK, vcos, vsin, v_interleaved, sink,
-                                                   keep, sig_bias);
+                                                   keep, sig_bias, chunk, maps, diff);
     return 0;
 }
 }  // namespace
 
 // Floats of workspace for a step of T single tokens whose longest request has max_kv_len keys
 // (0: such a step has one block of keys a row at most and needs none).
-extern "C" size_t ri_attention_window_workspace(int T, int H, int dk, int dv, int window, int max_kv_len, int keep) {
-    const int slots = aw_slots(dk, dv, window, max_kv_len, window > 0 ? keep : 0);
-    return slots <= 1 ? 0 : (size_t)T * H * slots * (dv + 2);
+extern "C" size_t ri_attention_window_workspace(int T, int H, int dv, int window, int chunk, int max_kv_len, int keep, int maps) {
+    const int slots = aw_slots(window, chunk, max_kv_len, keep);
+    return slots <= 1 ? 0 : (size_t)T * H * maps * slots * (dv + 2);
 }
 
 // Attention of the step's tokens (rotated queries in q) over the cache; out [T][>= H dv].
@@ -762,34 +857,39 @@ extern "C" size_t ri_attention_window_workspace(int T, int H, int dk, int dv, in
 // keep: with a window, the first `keep` positions of a request stay in sight of every later query.
 // sig_bias [H] (null: softmax): the weight of a visible key is sigmoid(score + sig_bias[head]) and the
 // weights are not normalised over the keys (no sink then).
+// chunk: a query sees keys of its own chunk of so many positions only (0: no chunks).
+// maps = 2: q [T][>= H 2 dk], keys of 2 dk features, sinks and biases [2 H]; a head's output is
+// gain (a - lam b) / rms(a - lam b) with a, b its two maps' outputs (diff_eps inside the root; no turned values then).
 extern "C" int ri_attention_window(
         const void* q, int q_stride, void* out, int out_stride, int dtype, const void* kc, const void* vc,
         int num_pages, int page, int H, int Hkv, int dk, int dv, const int* table, int max_blocks,
         const int* cu_q, const int* q_start, const int* kv_lens, int num_rows, int T,
         float scale, int window, const float* vcos, const float* vsin, int v_table_rows, int v_interleaved,
         int single_tokens, int max_kv_len, float* workspace, size_t workspace_floats, const float* sink,
-        int keep, const float* sig_bias, hipStream_t stream) {
-    RI_REQUIRE(ri_attention_window_supported(H, Hkv, dk, dv), "ri_attention_window: sizes not taken (H=%d Hkv=%d dk=%d dv=%d)", H, Hkv, dk, dv);
-    RI_REQUIRE(keep >= 0 && !(sink && sig_bias), "ri_attention_window: keep must be >= 0, and sigmoid weights take no sink");
-    if (window == 0) keep = 0;
+        int keep, const float* sig_bias, int chunk, int maps, float diff_lam, float diff_gain, float diff_eps, hipStream_t stream) {
+    RI_REQUIRE(ri_attention_window_supported(H, Hkv, dk, dv, maps), "ri_attention_window: sizes not taken (H=%d Hkv=%d dk=%d dv=%d maps=%d)", H, Hkv, dk, dv, maps);
+    RI_REQUIRE(keep >= 0 && chunk >= 0 && !(sink && sig_bias), "ri_attention_window: keep and chunk must be >= 0, and sigmoid weights take no sink");
+    RI_REQUIRE(maps == 1 || (!vcos && diff_eps > 0.f), "ri_attention_window: the difference of two maps takes no turned values and an eps > 0");
+    if (window == 0 && chunk == 0) keep = 0;
     RI_REQUIRE(T >= 0 && num_rows >= 0 && max_blocks > 0 && num_pages > 0 && window >= 0 && page > 0, "ri_attention_window: bad sizes");
-    RI_REQUIRE(q_stride >= H * dk && out_stride >= H * dv, "ri_attention_window: row strides too small");
+    RI_REQUIRE(q_stride >= H * maps * dk && out_stride >= H * dv, "ri_attention_window: row strides too small");
     if (vcos) RI_REQUIRE(vsin && dv % 2 == 0 && v_table_rows > 0, "ri_attention_window: a turned value needs an even size and both tables");
     if (T == 0 || num_rows == 0) return 0;
     RI_REQUIRE(q && out && kc && vc && table && cu_q && q_start && kv_lens, "ri_attention_window: null pointer");
     RI_REQUIRE(Hkv <= 65535, "ri_attention_window: too many key/value heads for the grid");
     int slots = 0;
     if (single_tokens && workspace && max_kv_len > 0) {
-        slots = aw_slots(dk, dv, window, max_kv_len, keep);
+        slots = aw_slots(window, chunk, max_kv_len, keep);
         if (slots <= 1) slots = 0;
-        else RI_REQUIRE(workspace_floats >= (size_t)T * H * slots * (dv + 2) && slots <= 65535 && num_rows <= 65535 && H <= 65535,
+        else RI_REQUIRE(workspace_floats >= (size_t)T * H * maps * slots * (dv + 2) && slots <= 65535 && num_rows <= 65535 && H <= 65535,
                         "ri_attention_window: workspace of %zu floats for %d slots, or too many rows for the grid", workspace_floats, slots);
     }
+    const DiffHow diff{diff_lam, diff_gain, diff_eps};
     int rc;
     if (dtype == RI_F32)
-        rc = aw_launch<float>((const float*)q, q_stride, (float*)out, out_stride, (const float*)kc, (const float*)vc, table, max_blocks, cu_q, q_start, kv_lens, num_rows, T, H, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, slots, workspace, sink, keep, sig_bias, stream);
+        rc = aw_launch<float>((const float*)q, q_stride, (float*)out, out_stride, (const float*)kc, (const float*)vc, table, max_blocks, cu_q, q_start, kv_lens, num_rows, T, H * maps, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, slots, workspace, sink, keep, sig_bias, chunk, maps, diff, stream);
     else if (dtype == RI_BF16)
-        rc = aw_launch<bf16_t>((const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)kc, (const bf16_t*)vc, table, max_blocks, cu_q, q_start, kv_lens, num_rows, T, H, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, slots, workspace, sink, keep, sig_bias, stream);
+        rc = aw_launch<bf16_t>((const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)kc, (const bf16_t*)vc, table, max_blocks, cu_q, q_start, kv_lens, num_rows, T, H * maps, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, slots, workspace, sink, keep, sig_bias, chunk, maps, diff, stream);
     else
         return ri_fail("ri_attention_window: unknown dtype %d", dtype);
     if (rc) return rc;
@@ -818,8 +918,8 @@ namespace {
 typedef float aw_f16 __attribute__((ext_vector_type(16)));
 constexpr int AM_KEYS = 64;      // keys a stage
 
-size_t am_lds_bytes(int QU, int dv) {
-    const size_t stage = (size_t)AM_KEYS * (8 * QU + 4) + (size_t)AM_KEYS * (dv + 8);
+size_t am_lds_bytes(int QU, int dv, int maps) {
+    const size_t stage = (size_t)AM_KEYS * (maps * 8 * QU + 4) + (size_t)AM_KEYS * (dv + 8);
     const size_t outs = (size_t)128 * dv;
     return sizeof(float) * (64 + (stage > outs ? stage : outs));
 }
@@ -831,12 +931,13 @@ __global__ __launch_bounds__(256) void attn_window_mfma_kernel(
         const int* __restrict__ cu_q, const int* __restrict__ q_start, const int* __restrict__ kv_lens,
         int num_rows, int H, int Hkv, int dk, int dv, int page, float scale, int window,
         const float* __restrict__ vcos, const float* __restrict__ vsin, int v_interleaved, const float* __restrict__ sink,
-        int keep, const float* __restrict__ sig_bias) {
+        int keep, const float* __restrict__ sig_bias, int chunk, int maps, DiffHow diff) {
     extern __shared__ __align__(16) float lds[];
-    constexpr int DKP = 8 * QU, KS = DKP + 4;
+    constexpr int DKP = 8 * QU;
+    const int KS = maps * DKP + 4, dkr = maps * dk;    // (maps = 2: map m of a key lies at m * DKP of its row)
     const int vs_stride = dv + 8;
     int* koff = reinterpret_cast<int*>(lds);           // [64]
-    float* Ks = lds + 64;                              // [64][DKP + 4]
+    float* Ks = lds + 64;                              // [64][maps DKP + 4]
     float* Vs = Ks + AM_KEYS * KS;                     // [64][dv + 8]
     float* Os = Ks;                                    // [4 waves][32][dv], after the last stage
 
@@ -859,16 +960,17 @@ __global__ __launch_bounds__(256) void attn_window_mfma_kernel(
     const int p0 = q_start[b] + (t0 - cu_q[b]);
     const int kv_len = kv_lens[b];
     const int blk_last = min(kv_len, p0 + nt);
-    const int blk_first = window > 0 ? max(0, p0 + 1 - window) : 0;
+    const int blk_first = aw_first_key(p0, window, chunk);
     // this wave's 32 tokens and head
     const int sub = wave / HB, hh = hgroup * 4 + wave % HB;
     const bool wave_on = sub < SB && hh < G && nt - 32 * sub > 0;
     const int t0w = t0 + 32 * sub, ntw = wave_on ? min(32, nt - 32 * sub) : 0, p0w = p0 + 32 * sub;
     const int head = g * G + (hh < G ? hh : 0);
     const int w_last = wave_on ? min(kv_len, p0w + ntw) : 0;
-    const int w_first = window > 0 ? max(0, p0w + 1 - window) : 0;
+    const int w_first = aw_first_key(p0w, window, chunk);
     const bool row_on = lq < ntw;
     const int pq = p0w + lq;                           // the lane's query position
+    const int q_first = aw_first_key(pq, window, chunk);
 
     // the query's features, in the order the products take them: unit u, step c -> feature 8 u + 4 lh + c
     float qr[QU * 4];
@@ -906,21 +1008,22 @@ __global__ __launch_bounds__(256) void attn_window_mfma_kernel(
         __syncthreads();
         constexpr int VL = 16 / sizeof(T);
         if (dk % VL == 0) {
-            const int pieces = dk / VL;
+            const int pieces = dkr / VL, a_map = dk / VL;
             for (int e = tid; e < AM_KEYS * pieces; e += 256) {
                 const int jj = e / pieces, pc = e - jj * pieces, off = koff[jj];
+                const int gap = pc >= a_map ? DKP - dk : 0;      // the second map's half begins at DKP
                 float f[VL];
 #pragma unroll
                 for (int u = 0; u < VL; ++u) f[u] = 0.f;
-                if (off >= 0) ld_vec16(kc + (size_t)off * dk + pc * VL, f);
+                if (off >= 0) ld_vec16(kc + (size_t)off * dkr + pc * VL, f);
 #pragma unroll
                 for (int u = 0; u < VL; u += 4)
-                    *reinterpret_cast<float4*>(Ks + jj * KS + pc * VL + u) = make_float4(f[u], f[u + 1], f[u + 2], f[u + 3]);
+                    *reinterpret_cast<float4*>(Ks + jj * KS + gap + pc * VL + u) = make_float4(f[u], f[u + 1], f[u + 2], f[u + 3]);
             }
         } else {
-            for (int e = tid; e < AM_KEYS * dk; e += 256) {
-                const int jj = e / dk, dd = e - jj * dk, off = koff[jj];
-                Ks[jj * KS + dd] = off >= 0 ? ld_f32(kc + (size_t)off * dk + dd) : 0.f;
+            for (int e = tid; e < AM_KEYS * dkr; e += 256) {
+                const int jj = e / dkr, dd = e - jj * dkr, off = koff[jj];
+                Ks[jj * KS + (dd >= dk ? DKP - dk : 0) + dd] = off >= 0 ? ld_f32(kc + (size_t)off * dkr + dd) : 0.f;
             }
         }
         if (page % VL == 0) {
@@ -955,7 +1058,7 @@ __global__ __launch_bounds__(256) void attn_window_mfma_kernel(
             aw_f16 s;
 #pragma unroll
             for (int i = 0; i < 16; ++i) s[i] = 0.f;
-            const float* krow = Ks + (32 * half + lq) * KS + 4 * lh;
+            const float* krow = Ks + (32 * half + lq) * KS + 4 * lh + (maps == 2 ? (wave & 1) * DKP : 0);      // (heads hh and wave: one parity)
 #pragma unroll
             for (int u = 0; u < QU; ++u) {
                 const float4 k4 = *reinterpret_cast<const float4*>(krow + 8 * u);
@@ -965,7 +1068,7 @@ __global__ __launch_bounds__(256) void attn_window_mfma_kernel(
                 s = __builtin_amdgcn_mfma_f32_32x32x2f32(k4.w, qr[u * 4 + 3], s, 0, 0, 0);
             }
             // register i: key kt0 + 8 (i / 4) + 4 lh + i % 4, for the lane's query
-            const int j_lo = window > 0 ? pq + 1 - window : 0, j_hi = min(pq + 1, kv_len);
+            const int j_lo = q_first, j_hi = min(pq + 1, kv_len);
             float mt = -INFINITY;
 #pragma unroll
             for (int i = 0; i < 16; ++i) {
@@ -1026,6 +1129,22 @@ __global__ __launch_bounds__(256) void attn_window_mfma_kernel(
     }
     __syncthreads();
     if (!wave_on) return;
+    if (maps == 2) {
+        // the wave and its neighbour hold the two maps of one head for the same 32 tokens: each writes every other token
+        constexpr int NC = (FT + 1) / 2;
+        const float* o1 = Os + (size_t)(wave & ~1) * 32 * dv, *o2 = o1 + (size_t)32 * dv;
+        for (int r = wave & 1; r < ntw; r += 2) {
+            float a[NC], bb[NC];
+#pragma unroll
+            for (int c = 0; c < NC; ++c) {
+                const int f = lane + 64 * c;
+                a[c] = f < dv ? o1[r * dv + f] : 0.f;
+                bb[c] = f < dv ? o2[r * dv + f] : 0.f;
+            }
+            aw_write_difference<T, NC>(out + (size_t)(t0w + r) * out_stride + head / 2 * dv, a, bb, dv, lane, diff);
+        }
+        return;
+    }
     const int vh = dv >> 1;
     for (int r = 0; r < ntw; ++r) {
         T* orow = out + (size_t)(t0w + r) * out_stride + head * dv;
@@ -1048,9 +1167,9 @@ template <typename T, int QU, int FT>
 int am_launch_as(const T* q, int q_stride, T* out, int out_stride, const T* kc, const T* vc, const int* table, int max_blocks,
                  const int* cu_q, const int* q_start, const int* kv_lens, int num_rows, int Tn, int H, int Hkv, int dk, int dv,
                  int page, float scale, int window, const float* vcos, const float* vsin, int v_interleaved, const float* sink,
-                 int keep, const float* sig_bias, hipStream_t stream) {
-    const int G = H / Hkv, HB = G < 4 ? G : 4, SB = 4 / HB, TQB = 32 * SB;
-    const size_t lds = am_lds_bytes(QU, dv);
+                 int keep, const float* sig_bias, int chunk, int maps, DiffHow diff, hipStream_t stream) {
+    const int G = H / Hkv, HB = G < 4 ? G : 4, SB = 4 / HB, TQB = 32 * SB;      // (H: the maps of all heads)
+    const size_t lds = am_lds_bytes(QU, dv, maps);
     auto kernel = attn_window_mfma_kernel<T, QU, FT>;
     if (lds > 64 * 1024) {
         static bool asked = false;
@@ -1062,7 +1181,7 @@ int am_launch_as(const T* q, int q_stride, T* out, int out_stride, const T* kc, 
     }
     const int tiles = (Tn + TQB - 1) / TQB + num_rows;
     kernel<<<dim3(tiles, Hkv, (G + 3) / 4), 256, lds, stream>>>(q, q_stride, out, out_stride, kc, vc, table, max_blocks, cu_q, q_start,
-                                                               kv_lens, num_rows, H, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, sink, keep, sig_bias);
+                                                               kv_lens, num_rows, H, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, sink, keep, sig_bias, chunk, maps, diff);
     return 0;
 }
 
@@ -1070,9 +1189,9 @@ template <typename T>
 int am_launch(const T* q, int q_stride, T* out, int out_stride, const T* kc, const T* vc, const int* table, int max_blocks,
               const int* cu_q, const int* q_start, const int* kv_lens, int num_rows, int Tn, int H, int Hkv, int dk, int dv,
               int page, float scale, int window, const float* vcos, const float* vsin, int v_interleaved, const float* sink,
-              int keep, const float* sig_bias, hipStream_t stream) {
+              int keep, const float* sig_bias, int chunk, int maps, DiffHow diff, hipStream_t stream) {
 #define RI_AM(QU, FT) return am_launch_as<T, QU, FT>(q, q_stride, out, out_stride, kc, vc, table, max_blocks, cu_q, q_start, kv_lens, \
-        num_rows, Tn, H, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, sink, keep, sig_bias, stream)
+        num_rows, Tn, H, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, sink, keep, sig_bias, chunk, maps, diff, stream)
     if (dk <= 64) { if (dv <= 64) RI_AM(8, 2); if (dv <= 128) RI_AM(8, 4); RI_AM(8, 8); }
     if (dk <= 128) { if (dv <= 64) RI_AM(16, 2); if (dv <= 128) RI_AM(16, 4); RI_AM(16, 8); }
     if (dv <= 64) RI_AM(32, 2);
@@ -1083,10 +1202,10 @@ int am_launch(const T* q, int q_stride, T* out, int out_stride, const T* kc, con
 
 }  // namespace
 
-extern "C" int ri_attention_window_mfma_supported(int H, int Hkv, int dk, int dv) {
-    if (!ri_attention_window_supported(H, Hkv, dk, dv)) return 0;
+extern "C" int ri_attention_window_mfma_supported(int H, int Hkv, int dk, int dv, int maps) {
+    if (!ri_attention_window_supported(H, Hkv, dk, dv, maps)) return 0;
     const int QU = dk <= 64 ? 8 : dk <= 128 ? 16 : 32;
-    return am_lds_bytes(QU, dv) <= 160 * 1024;
+    return am_lds_bytes(QU, dv, maps) <= 160 * 1024;
 }
 
 // The same attention as ri_attention_window for steps with prompt portions, on the 32-bit matrix
@@ -1096,21 +1215,24 @@ extern "C" int ri_attention_window_mfma(
         int num_pages, int page, int H, int Hkv, int dk, int dv, const int* table, int max_blocks,
         const int* cu_q, const int* q_start, const int* kv_lens, int num_rows, int T,
         float scale, int window, const float* vcos, const float* vsin, int v_table_rows, int v_interleaved,
-        const float* sink, int keep, const float* sig_bias, hipStream_t stream) {
-    RI_REQUIRE(ri_attention_window_mfma_supported(H, Hkv, dk, dv), "ri_attention_window_mfma: sizes not taken (H=%d Hkv=%d dk=%d dv=%d)", H, Hkv, dk, dv);
-    RI_REQUIRE(keep >= 0 && !(sink && sig_bias), "ri_attention_window_mfma: keep must be >= 0, and sigmoid weights take no sink");
-    if (window == 0) keep = 0;
+        const float* sink, int keep, const float* sig_bias, int chunk, int maps, float diff_lam, float diff_gain, float diff_eps,
+        hipStream_t stream) {
+    RI_REQUIRE(ri_attention_window_mfma_supported(H, Hkv, dk, dv, maps), "ri_attention_window_mfma: sizes not taken (H=%d Hkv=%d dk=%d dv=%d maps=%d)", H, Hkv, dk, dv, maps);
+    RI_REQUIRE(keep >= 0 && chunk >= 0 && !(sink && sig_bias), "ri_attention_window_mfma: keep and chunk must be >= 0, and sigmoid weights take no sink");
+    RI_REQUIRE(maps == 1 || (!vcos && diff_eps > 0.f), "ri_attention_window_mfma: the difference of two maps takes no turned values and an eps > 0");
+    if (window == 0 && chunk == 0) keep = 0;
     RI_REQUIRE(T >= 0 && num_rows >= 0 && max_blocks > 0 && num_pages > 0 && window >= 0 && page > 0, "ri_attention_window_mfma: bad sizes");
-    RI_REQUIRE(q_stride >= H * dk && out_stride >= H * dv, "ri_attention_window_mfma: row strides too small");
+    RI_REQUIRE(q_stride >= H * maps * dk && out_stride >= H * dv, "ri_attention_window_mfma: row strides too small");
     if (vcos) RI_REQUIRE(vsin && dv % 2 == 0 && v_table_rows > 0, "ri_attention_window_mfma: a turned value needs an even size and both tables");
     if (T == 0 || num_rows == 0) return 0;
     RI_REQUIRE(q && out && kc && vc && table && cu_q && q_start && kv_lens, "ri_attention_window_mfma: null pointer");
     RI_REQUIRE(Hkv <= 65535, "ri_attention_window_mfma: too many key/value heads for the grid");
+    const DiffHow diff{diff_lam, diff_gain, diff_eps};
     int rc;
     if (dtype == RI_F32)
-        rc = am_launch<float>((const float*)q, q_stride, (float*)out, out_stride, (const float*)kc, (const float*)vc, table, max_blocks, cu_q, q_start, kv_lens, num_rows, T, H, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, sink, keep, sig_bias, stream);
+        rc = am_launch<float>((const float*)q, q_stride, (float*)out, out_stride, (const float*)kc, (const float*)vc, table, max_blocks, cu_q, q_start, kv_lens, num_rows, T, H * maps, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, sink, keep, sig_bias, chunk, maps, diff, stream);
     else if (dtype == RI_BF16)
-        rc = am_launch<bf16_t>((const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)kc, (const bf16_t*)vc, table, max_blocks, cu_q, q_start, kv_lens, num_rows, T, H, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, sink, keep, sig_bias, stream);
+        rc = am_launch<bf16_t>((const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)kc, (const bf16_t*)vc, table, max_blocks, cu_q, q_start, kv_lens, num_rows, T, H * maps, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, sink, keep, sig_bias, chunk, maps, diff, stream);
     else
         return ri_fail("ri_attention_window_mfma: unknown dtype %d", dtype);
     if (rc) return rc;

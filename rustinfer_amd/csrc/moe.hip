@@ -12,6 +12,11 @@
 //                       weights by a constant.  Fs more columns after the experts' are a shared expert that
 //                       every token uses with weight 1: act[t][E F + i] = silu(gu[t][2 E F + i]) * gu[t][2 E F + Fs + i];
 //                       columns beyond E F + Fs up to the width given are zeros.
+//                       The activation of a pair (g, u) of gate and up values may also be the clipped one:
+//                       g' = min(g, limit), u' = clamp(u, -limit, limit), g' sigmoid(slope g') (u' + shift), with a
+//                       limit of its own for the shared expert; the weight may multiply the expert's INPUT instead
+//                       of its output (both of its pre-activations, then, since they are linear in it); and
+//                       one more logit a token may gate the shared expert (its sigmoid in place of weight 1).
 //   moe_swiglu_routed   the two in one launch: every block makes its token's weights from the logits
 //                       itself (what the engine runs; the two above are its halves, kept for callers
 //                       that want the weights).
@@ -83,12 +88,31 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict_
     route_token(logits + (size_t)t * l_stride, weights + (size_t)t * E, E, top, how, lane);
 }
 
-// column i of the shared expert's activation from its gate and up columns [gate Fs | up Fs]; 0 beyond Fs
+// What an expert does with its gate and up values, and where its weight goes.
+struct ActHow {
+    int clipped;              // 0: silu(g) u;  1: the clipped form
+    float limit, shared_limit, slope, shift;
+    int weigh_input;          // the weight multiplies g and u (the expert's input), not the result
+};
+
+__device__ __forceinline__ float gated_pair(float g, float u, const ActHow& how, float limit) {
+    if (!how.clipped) return (g / (1.f + expf(-g))) * u;
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    return (g / (1.f + expf(-how.slope * g))) * (u + how.shift);
+}
+
+__device__ __forceinline__ float weighted_pair(float wgt, float g, float u, const ActHow& how) {
+    return how.weigh_input ? gated_pair(wgt * g, wgt * u, how, how.limit) : wgt * gated_pair(g, u, how, how.limit);
+}
+
+// column i of the shared expert's activation from its gate and up columns [gate Fs | up Fs]; 0 beyond Fs.
+// gate: the logit of its own gate, or null
 template <typename T>
-__device__ __forceinline__ float shared_column(const T* __restrict__ row, int i, int Fs) {
+__device__ __forceinline__ float shared_column(const T* __restrict__ row, int i, int Fs, const ActHow& how, const float* __restrict__ gate) {
     if (i >= Fs) return 0.f;
-    const float g = ld_f32(row + i), u = ld_f32(row + Fs + i);
-    return (g / (1.f + expf(-g))) * u;
+    const float y = gated_pair(ld_f32(row + i), ld_f32(row + Fs + i), how, how.shared_limit);
+    return gate ? y / (1.f + expf(-*gate)) : y;
 }
 
 // moe_swiglu_weighted with the routing done on the way: the block's first wave makes the token's weights
@@ -96,39 +120,41 @@ __device__ __forceinline__ float shared_column(const T* __restrict__ row, int i,
 template <typename T>
 __global__ __launch_bounds__(256) void moe_swiglu_routed_kernel(const T* __restrict__ gu, int gu_stride, const float* __restrict__ logits,
                                                                int l_stride, T* __restrict__ act, int act_stride, int E, int F,
-                                                               int top, RouteHow how, int Fs, int width) {
+                                                               int top, RouteHow how, int Fs, int width, ActHow ah,
+                                                               const float* __restrict__ sg, int sg_stride) {
     __shared__ float wts[64 * MOE_EPL];
     const int t = blockIdx.y;
     if (threadIdx.x < 64) route_token(logits + (size_t)t * l_stride, wts, E, top, how, threadIdx.x);
     __syncthreads();
     const int idx = blockIdx.x * 256 + threadIdx.x;
     if (idx >= width) return;
-    if (idx >= E * F) { st_f32(act + (size_t)t * act_stride + idx, shared_column(gu + (size_t)t * gu_stride + (size_t)E * 2 * F, idx - E * F, Fs)); return; }
+    if (idx >= E * F) { st_f32(act + (size_t)t * act_stride + idx, shared_column(gu + (size_t)t * gu_stride + (size_t)E * 2 * F, idx - E * F, Fs, ah, sg ? sg + (size_t)t * sg_stride : nullptr)); return; }
     const int e = idx / F, i = idx - e * F;
     const float wgt = wts[e];
     float y = 0.f;
     if (wgt != 0.f) {
         const T* row = gu + (size_t)t * gu_stride + (size_t)e * 2 * F;
         const float g = ld_f32(row + i), u = ld_f32(row + F + i);
-        y = wgt * (g / (1.f + expf(-g))) * u;
+        y = weighted_pair(wgt, g, u, ah);
     }
     st_f32(act + (size_t)t * act_stride + idx, y);
 }
 
 template <typename T>
 __global__ __launch_bounds__(256) void moe_swiglu_weighted_kernel(const T* __restrict__ gu, int gu_stride, const float* __restrict__ weights,
-                                                                 T* __restrict__ act, int act_stride, int E, int F, int Fs, int width) {
+                                                                 T* __restrict__ act, int act_stride, int E, int F, int Fs, int width, ActHow ah,
+                                                                 const float* __restrict__ sg, int sg_stride) {
     const int t = blockIdx.y;
     const int idx = blockIdx.x * 256 + threadIdx.x;
     if (idx >= width) return;
-    if (idx >= E * F) { st_f32(act + (size_t)t * act_stride + idx, shared_column(gu + (size_t)t * gu_stride + (size_t)E * 2 * F, idx - E * F, Fs)); return; }
+    if (idx >= E * F) { st_f32(act + (size_t)t * act_stride + idx, shared_column(gu + (size_t)t * gu_stride + (size_t)E * 2 * F, idx - E * F, Fs, ah, sg ? sg + (size_t)t * sg_stride : nullptr)); return; }
     const int e = idx / F, i = idx - e * F;
     const float wgt = weights[(size_t)t * E + e];
     float y = 0.f;
     if (wgt != 0.f) {
         const T* row = gu + (size_t)t * gu_stride + (size_t)e * 2 * F;
         const float g = ld_f32(row + i), u = ld_f32(row + F + i);
-        y = wgt * (g / (1.f + expf(-g))) * u;
+        y = weighted_pair(wgt, g, u, ah);
     }
     st_f32(act + (size_t)t * act_stride + idx, y);
 }
@@ -152,47 +178,44 @@ extern "C" int ri_moe_route(const float* logits, int l_stride, float* weights, i
 }
 
 // Fs: columns of a shared expert behind the experts' (0: none); width: columns of act that are written
-// (E F + Fs of activations, zeros beyond).
-extern "C" int ri_moe_swiglu_weighted_shared(const void* gu, int gu_stride, const float* weights, void* act, int act_stride, int dtype,
-                                             int T, int E, int F, int Fs, int width, hipStream_t stream) {
+// (E F + Fs of activations, zeros beyond).  clipped, limit, shared_limit, slope, shift, weigh_input: see ActHow.
+// sg (null: none): 32-bit logits of the shared expert's gate, token t's at sg[t * sg_stride].
+extern "C" int ri_moe_act_weighted(const void* gu, int gu_stride, const float* weights, void* act, int act_stride, int dtype,
+                                   int T, int E, int F, int Fs, int width, int clipped, float limit, float shared_limit,
+                                   float slope, float shift, int weigh_input, const float* sg, int sg_stride, hipStream_t stream) {
     RI_REQUIRE(T >= 0 && E > 0 && F > 0 && Fs >= 0 && width >= E * F + Fs && gu_stride >= 2 * E * F + 2 * Fs && act_stride >= width,
-               "ri_moe_swiglu_weighted: bad sizes");
+               "ri_moe_act_weighted: bad sizes");
+    RI_REQUIRE(!sg || sg_stride > 0, "ri_moe_act_weighted: the shared gate's logits need a stride");
     if (T == 0) return 0;
-    RI_REQUIRE(gu && weights && act, "ri_moe_swiglu_weighted: null pointer");
-    RI_REQUIRE(T <= 65535, "ri_moe_swiglu_weighted: too many rows for the grid");
+    RI_REQUIRE(gu && weights && act, "ri_moe_act_weighted: null pointer");
+    RI_REQUIRE(T <= 65535, "ri_moe_act_weighted: too many rows for the grid");
     const dim3 grid((width + 255) / 256, T);
-    if (dtype == RI_F32) moe_swiglu_weighted_kernel<float><<<grid, 256, 0, stream>>>((const float*)gu, gu_stride, weights, (float*)act, act_stride, E, F, Fs, width);
-    else if (dtype == RI_BF16) moe_swiglu_weighted_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)gu, gu_stride, weights, (bf16_t*)act, act_stride, E, F, Fs, width);
-    else return ri_fail("ri_moe_swiglu_weighted: unknown dtype %d", dtype);
-    RI_LAUNCHED("ri_moe_swiglu_weighted");
+    const ActHow ah{clipped, limit, shared_limit, slope, shift, weigh_input};
+    if (dtype == RI_F32) moe_swiglu_weighted_kernel<float><<<grid, 256, 0, stream>>>((const float*)gu, gu_stride, weights, (float*)act, act_stride, E, F, Fs, width, ah, sg, sg_stride);
+    else if (dtype == RI_BF16) moe_swiglu_weighted_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)gu, gu_stride, weights, (bf16_t*)act, act_stride, E, F, Fs, width, ah, sg, sg_stride);
+    else return ri_fail("ri_moe_act_weighted: unknown dtype %d", dtype);
+    RI_LAUNCHED("ri_moe_act_weighted");
     return 0;
-}
-
-extern "C" int ri_moe_swiglu_weighted(const void* gu, int gu_stride, const float* weights, void* act, int act_stride, int dtype,
-                                      int T, int E, int F, hipStream_t stream) {
-    return ri_moe_swiglu_weighted_shared(gu, gu_stride, weights, act, act_stride, dtype, T, E, F, 0, E * F, stream);
 }
 
 // The two in one launch: act from gate_up and the router's 32-bit logits [T][>= E].
-extern "C" int ri_moe_swiglu_routed_as(const void* gu, int gu_stride, const float* logits, int l_stride, void* act, int act_stride,
-                                       int dtype, int T, int E, int F, int top, int renorm, int sigmoid, float eps, float scale,
-                                       int Fs, int width, hipStream_t stream) {
+extern "C" int ri_moe_act_routed(const void* gu, int gu_stride, const float* logits, int l_stride, void* act, int act_stride,
+                                 int dtype, int T, int E, int F, int top, int renorm, int sigmoid, float eps, float scale,
+                                 int Fs, int width, int clipped, float limit, float shared_limit, float slope, float shift,
+                                 int weigh_input, const float* sg, int sg_stride, hipStream_t stream) {
     RI_REQUIRE(T >= 0 && E > 0 && F > 0 && Fs >= 0 && width >= E * F + Fs && gu_stride >= 2 * E * F + 2 * Fs && act_stride >= width && l_stride >= E,
-               "ri_moe_swiglu_routed: bad sizes");
-    RI_REQUIRE(top > 0 && top <= E && E <= 64 * MOE_EPL, "ri_moe_swiglu_routed: top %d of %d experts (up to %d)", top, E, 64 * MOE_EPL);
+               "ri_moe_act_routed: bad sizes");
+    RI_REQUIRE(top > 0 && top <= E && E <= 64 * MOE_EPL, "ri_moe_act_routed: top %d of %d experts (up to %d)", top, E, 64 * MOE_EPL);
+    RI_REQUIRE(!sg || sg_stride > 0, "ri_moe_act_routed: the shared gate's logits need a stride");
     if (T == 0) return 0;
-    RI_REQUIRE(gu && logits && act, "ri_moe_swiglu_routed: null pointer");
-    RI_REQUIRE(T <= 65535, "ri_moe_swiglu_routed: too many rows for the grid");
+    RI_REQUIRE(gu && logits && act, "ri_moe_act_routed: null pointer");
+    RI_REQUIRE(T <= 65535, "ri_moe_act_routed: too many rows for the grid");
     const dim3 grid((width + 255) / 256, T);
     const RouteHow how{sigmoid, renorm, eps, scale};
-    if (dtype == RI_F32) moe_swiglu_routed_kernel<float><<<grid, 256, 0, stream>>>((const float*)gu, gu_stride, logits, l_stride, (float*)act, act_stride, E, F, top, how, Fs, width);
-    else if (dtype == RI_BF16) moe_swiglu_routed_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)gu, gu_stride, logits, l_stride, (bf16_t*)act, act_stride, E, F, top, how, Fs, width);
-    else return ri_fail("ri_moe_swiglu_routed: unknown dtype %d", dtype);
-    RI_LAUNCHED("ri_moe_swiglu_routed");
+    const ActHow ah{clipped, limit, shared_limit, slope, shift, weigh_input};
+    if (dtype == RI_F32) moe_swiglu_routed_kernel<float><<<grid, 256, 0, stream>>>((const float*)gu, gu_stride, logits, l_stride, (float*)act, act_stride, E, F, top, how, Fs, width, ah, sg, sg_stride);
+    else if (dtype == RI_BF16) moe_swiglu_routed_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)gu, gu_stride, logits, l_stride, (bf16_t*)act, act_stride, E, F, top, how, Fs, width, ah, sg, sg_stride);
+    else return ri_fail("ri_moe_act_routed: unknown dtype %d", dtype);
+    RI_LAUNCHED("ri_moe_act_routed");
     return 0;
-}
-
-extern "C" int ri_moe_swiglu_routed(const void* gu, int gu_stride, const float* logits, int l_stride, void* act, int act_stride,
-                                    int dtype, int T, int E, int F, int top, int renorm, hipStream_t stream) {
-    return ri_moe_swiglu_routed_as(gu, gu_stride, logits, l_stride, act, act_stride, dtype, T, E, F, top, renorm, 0, 0.f, 1.f, 0, E * F, stream);
 }

@@ -1001,15 +1001,16 @@ def rotate_kv_write(q: torch.Tensor, k: Optional[torch.Tensor], v: Optional[torc
 WINDOW_ATTENTION_MFMA = True     # steps with prompt portions take the matrix-instruction kernel (False: the FMA one, for comparison)
 
 
-def window_attention_supported(H: int, Hkv: int, dk: int, dv: int) -> bool:
-    return bool(_lib().ri_attention_window_supported(H, Hkv, dk, dv))
+def window_attention_supported(H: int, Hkv: int, dk: int, dv: int, maps: int = 1) -> bool:
+    return bool(_lib().ri_attention_window_supported(H, Hkv, dk, dv, maps))
 
 
 def window_attention(q: torch.Tensor, out: torch.Tensor, H: int, Hkv: int, dk: int, dv: int,
                      k_cache: torch.Tensor, v_cache: torch.Tensor, block_table: torch.Tensor, page: int,
                      ctx, scale: float, window: int = 0, value_rotary=None,
                      interleaved_values: bool = False, sink: Optional[torch.Tensor] = None,
-                     keep_first: int = 0, sigmoid_bias: Optional[torch.Tensor] = None) -> None:
+                     keep_first: int = 0, sigmoid_bias: Optional[torch.Tensor] = None, chunk: int = 0,
+                     difference=None) -> None:
     """Attention of the step's tokens (rotated queries ``q [T, H dk]``) over the cache into
     ``out [T, H dv]``: keys of size ``dk``, values of size ``dv``, the last ``window`` positions
     (0: all).  ``value_rotary``: the cached values are turned by their positions, and each sum is
@@ -1017,19 +1018,27 @@ def window_attention(q: torch.Tensor, out: torch.Tensor, H: int, Hkv: int, dk: i
     softmax's denominator, with no key and no value.  ``keep_first``: with a window, the first so many
     positions of a request stay in sight of every later query.  ``sigmoid_bias`` (32-bit, one number a
     query head): no softmax; a visible key's weight is ``sigmoid(score + sigmoid_bias[h])``, and the
-    weights are not normalised over the keys."""
+    weights are not normalised over the keys.  ``chunk``: a query sees keys of its own chunk of so many
+    positions only, counted from the request's first.  ``difference = (lam, gain, eps)``: every query head
+    holds two queries and every key head two keys of ``dk`` features side by side (``q [T, H 2 dk]``, keys of
+    ``2 dk``) over one value; with the two maps' outputs ``a``, ``b`` (32-bit) a head's output is
+    ``gain (a - lam b) / sqrt(mean((a - lam b)^2) + eps)``."""
     _dev(q, out, k_cache, v_cache, block_table, sink, sigmoid_bias)
-    _f32_vec(sink, H, "window_attention: the sink")
-    _f32_vec(sigmoid_bias, H, "window_attention: the sigmoids' bias")
+    maps = 2 if difference is not None else 1
+    lam, gain, diff_eps = (ctypes.c_float(v) for v in (difference if difference is not None else (0.0, 1.0, 1.0)))
+    if difference is not None and value_rotary is not None:
+        raise KernelError("window_attention: the difference of two maps takes no turned values")
+    _f32_vec(sink, H * maps, "window_attention: the sink")
+    _f32_vec(sigmoid_bias, H * maps, "window_attention: the sigmoids' bias")
     if sink is not None and sigmoid_bias is not None:
         raise KernelError("window_attention: sigmoid weights take no sink")
-    keep_first = int(keep_first) if window else 0
+    keep_first = int(keep_first) if window or chunk else 0
     _rows2d(q, "q")
     _rows2d(out, "out")
     T = q.shape[0]
-    if q.shape[1] != H * dk or tuple(out.shape) != (T, H * dv) or out.dtype != q.dtype:
-        raise KernelError(f"window_attention: q must be [T, {H * dk}] and out [T, {H * dv}] of one dtype")
-    _check_cache_kv(k_cache, v_cache, Hkv, dk, dv, page, q.dtype, "window_attention")
+    if q.shape[1] != H * maps * dk or tuple(out.shape) != (T, H * dv) or out.dtype != q.dtype:
+        raise KernelError(f"window_attention: q must be [T, {H * maps * dk}] and out [T, {H * dv}] of one dtype")
+    _check_cache_kv(k_cache, v_cache, Hkv, maps * dk, dv, page, q.dtype, "window_attention")
     _i32(block_table, "block_table")
     if block_table.dim() != 2 or block_table.shape[0] < ctx.num_rows:
         raise KernelError("window_attention: block_table must be [rows, max_blocks]")
@@ -1038,26 +1047,27 @@ def window_attention(q: torch.Tensor, out: torch.Tensor, H: int, Hkv: int, dk: i
     _i32(ctx.kv_lens, "kv_lens", ctx.num_rows)
     vcos, vsin, vrows = _rot_tables(value_rotary, dv, "window_attention (values)")
     lib = _lib()
-    if ctx.max_q_len > 1 and WINDOW_ATTENTION_MFMA and lib.ri_attention_window_mfma_supported(H, Hkv, dk, dv):
+    if ctx.max_q_len > 1 and WINDOW_ATTENTION_MFMA and lib.ri_attention_window_mfma_supported(H, Hkv, dk, dv, maps):
         # steps with prompt portions: both products on the 32-bit matrix instructions
         _check(lib.ri_attention_window_mfma(
             _ptr(q), q.stride(0), _ptr(out), out.stride(0), _dt(q), _ptr(k_cache), _ptr(v_cache), k_cache.shape[0], page,
             H, Hkv, dk, dv, _ptr(block_table), block_table.shape[1], _ptr(ctx.cu_q), _ptr(ctx.q_start), _ptr(ctx.kv_lens),
             ctx.num_rows, T, ctypes.c_float(scale), int(window), vcos, vsin, vrows, int(bool(interleaved_values)), _ptr(sink),
-            keep_first, _ptr(sigmoid_bias), _stream()))
+            keep_first, _ptr(sigmoid_bias), int(chunk), maps, lam, gain, diff_eps, _stream()))
         return
     # a step of single tokens divides each row's keys between blocks, through a workspace
     single, ws, need = int(ctx.max_q_len == 1 and T <= ctx.num_rows), None, 0
     if single:
         lib.ri_attention_window_workspace.restype = ctypes.c_size_t
-        need = lib.ri_attention_window_workspace(T, H, dk, dv, int(window), int(ctx.max_kv_len), keep_first)
+        need = lib.ri_attention_window_workspace(T, H, dv, int(window), int(chunk), int(ctx.max_kv_len), keep_first, maps)
         if need:
             ws = ctx.workspace.get("attn.window_partials", need, 1, torch.float32)
     _check(lib.ri_attention_window(
         _ptr(q), q.stride(0), _ptr(out), out.stride(0), _dt(q), _ptr(k_cache), _ptr(v_cache), k_cache.shape[0], page,
         H, Hkv, dk, dv, _ptr(block_table), block_table.shape[1], _ptr(ctx.cu_q), _ptr(ctx.q_start), _ptr(ctx.kv_lens),
         ctx.num_rows, T, ctypes.c_float(scale), int(window), vcos, vsin, vrows, int(bool(interleaved_values)),
-        single, int(ctx.max_kv_len), _ptr(ws), ctypes.c_size_t(need), _ptr(sink), keep_first, _ptr(sigmoid_bias), _stream()))
+        single, int(ctx.max_kv_len), _ptr(ws), ctypes.c_size_t(need), _ptr(sink), keep_first, _ptr(sigmoid_bias),
+        int(chunk), maps, lam, gain, diff_eps, _stream()))
 
 
 # ---------------------------------------------------------------------------
@@ -1147,16 +1157,18 @@ def head_norm_kv_write(q: torch.Tensor, k: Optional[torch.Tensor], v: Optional[t
                        dk: int, dv: int, q_weight: Optional[torch.Tensor], k_weight: Optional[torch.Tensor],
                        eps: float, positions: torch.Tensor, row_of_token: torch.Tensor, k_cache: torch.Tensor,
                        v_cache: torch.Tensor, block_table: torch.Tensor, page: int, write_kv: bool = True,
-                       norm: bool = True, temp_coef: float = 0.0, temp_every: int = 0) -> None:
+                       norm: bool = True, temp_coef: float = 0.0, temp_every: int = 0, maps: int = 1) -> None:
     """Every head of ``q [T, H dk]`` and ``k [T, Hkv dk]`` divided by its root mean square
     (``norm``), times a 32-bit weight of ``dk`` entries shared by the heads (or None); the query at
     position p also times ``1 + temp_coef ln(floor((p + 1) / temp_every) + 1)`` (``temp_every > 0``).
-    q in place; k and ``v [T, Hkv dv]`` go into the token's page (``write_kv``)."""
+    q in place; k and ``v [T, Hkv dv]`` go into the token's page (``write_kv``).  ``maps``: a head holds so
+    many queries or keys of ``dk`` features side by side (``q [T, H maps dk]``, ``k [T, Hkv maps dk]``), each
+    normed on its own."""
     _dev(q, k, v, q_weight, k_weight, positions, row_of_token, k_cache, v_cache, block_table)
     _rows2d(q, "q")
     T = q.shape[0]
-    if q.shape[1] != H * dk:
-        raise KernelError(f"head_norm_kv_write: q must be [T, {H * dk}]")
+    if q.shape[1] != H * maps * dk:
+        raise KernelError(f"head_norm_kv_write: q must be [T, {H * maps * dk}]")
     _i32(positions, "positions", T)
     _i32(row_of_token, "row_of_token", T)
     _f32_vec(q_weight, dk, "head_norm_kv_write: the query weight")
@@ -1164,9 +1176,9 @@ def head_norm_kv_write(q: torch.Tensor, k: Optional[torch.Tensor], v: Optional[t
     if write_kv:
         _rows2d(k, "k")
         _rows2d(v, "v")
-        if tuple(k.shape) != (T, Hkv * dk) or tuple(v.shape) != (T, Hkv * dv) or k.dtype != q.dtype or v.dtype != q.dtype:
-            raise KernelError(f"head_norm_kv_write: k must be [T, {Hkv * dk}] and v [T, {Hkv * dv}] of {q.dtype}")
-        _check_cache_kv(k_cache, v_cache, Hkv, dk, dv, page, q.dtype, "head_norm_kv_write")
+        if tuple(k.shape) != (T, Hkv * maps * dk) or tuple(v.shape) != (T, Hkv * dv) or k.dtype != q.dtype or v.dtype != q.dtype:
+            raise KernelError(f"head_norm_kv_write: k must be [T, {Hkv * maps * dk}] and v [T, {Hkv * dv}] of {q.dtype}")
+        _check_cache_kv(k_cache, v_cache, Hkv, maps * dk, dv, page, q.dtype, "head_norm_kv_write")
         _i32(block_table, "block_table")
         if block_table.dim() != 2:
             raise KernelError("head_norm_kv_write: block_table must be [rows, max_blocks]")
@@ -1176,7 +1188,7 @@ def head_norm_kv_write(q: torch.Tensor, k: Optional[torch.Tensor], v: Optional[t
         _ptr(q_weight), _ptr(k_weight), int(bool(norm)), ctypes.c_float(eps), ctypes.c_float(temp_coef), int(temp_every),
         _ptr(positions), _ptr(row_of_token), _ptr(k_cache), _ptr(v_cache), k_cache.shape[0] if k_cache is not None else 0,
         _ptr(block_table), block_table.shape[1] if block_table is not None and block_table.dim() == 2 else 0, page,
-        int(bool(write_kv)), _stream()))
+        int(bool(write_kv)), int(maps), _stream()))
 
 
 def latent_kv_write(q: torch.Tensor, down: torch.Tensor, q_abs: torch.Tensor, H: int, d: int, r: int, R: int,
@@ -1262,37 +1274,60 @@ def moe_route(logits: torch.Tensor, weights: torch.Tensor, top: int, renormalize
                                   _score_kind(score), ctypes.c_float(norm_eps), ctypes.c_float(scale), _stream()))
 
 
+class ClippedGate:
+    """The experts' activation ``g' sigmoid(slope g') (u' + shift)`` with ``g' = min(g, limit)`` and
+    ``u' = clamp(u, -limit, limit)``; ``shared_limit`` is the shared expert's limit."""
+
+    def __init__(self, limit: float, shared_limit: Optional[float] = None, slope: float = 1.702, shift: float = 1.0):
+        self.limit, self.slope, self.shift = float(limit), float(slope), float(shift)
+        self.shared_limit = float(limit if shared_limit is None else shared_limit)
+
+
+def _act_args(clip: Optional[ClippedGate], weigh_input: bool, shared_gate: Optional[torch.Tensor], T: int, who: str):
+    f = ctypes.c_float
+    if shared_gate is not None and (shared_gate.dim() != 1 or shared_gate.shape[0] != T or shared_gate.dtype != torch.float32):
+        raise KernelError(f"{who}: one 32-bit logit a token expected for the shared expert's gate")
+    how = (0, f(0), f(0), f(0), f(0)) if clip is None else (1, f(clip.limit), f(clip.shared_limit), f(clip.slope), f(clip.shift))
+    return how + (int(bool(weigh_input)), _ptr(shared_gate), shared_gate.stride(0) if shared_gate is not None else 0)
+
+
 def moe_swiglu_weighted(gate_up: torch.Tensor, weights: torch.Tensor, act: torch.Tensor, E: int, F: int,
-                        shared: int = 0) -> None:
+                        shared: int = 0, clip: Optional[ClippedGate] = None, weigh_input: bool = False,
+                        shared_gate: Optional[torch.Tensor] = None) -> None:
     """``act[t, e F + i] = weights[t, e] * silu(gate_up[t, e 2F + i]) * gate_up[t, e 2F + F + i]``.
     ``shared`` > 0: ``gate_up`` has ``2 shared`` more columns, a shared expert's gate and up, and ``act`` gets
-    ``silu(gate) * up`` of them behind the experts' columns (weight 1); wider ``act``: zeros beyond."""
-    _dev(gate_up, weights, act)
+    ``silu(gate) * up`` of them behind the experts' columns (weight 1, or the sigmoid of ``shared_gate [T]``, 32-bit
+    logits of any stride); wider ``act``: zeros beyond.  ``clip``: the clipped activation instead of silu times
+    up.  ``weigh_input``: the weight multiplies an expert's gate and up values (its input) instead of the result."""
+    _dev(gate_up, weights, act, shared_gate)
     _rows2d(gate_up, "gate_up")
     _rows2d(act, "act")
     T, width = _moe_widths(gate_up, act, E, F, shared, "moe_swiglu_weighted")
     if weights.dtype != torch.float32 or tuple(weights.shape) != (T, E) or not weights.is_contiguous():
         raise KernelError("moe_swiglu_weighted: contiguous 32-bit weights [T, E] expected")
-    _check(_lib().ri_moe_swiglu_weighted_shared(_ptr(gate_up), gate_up.stride(0), _ptr(weights), _ptr(act), act.stride(0),
-                                                _dt(act), T, E, F, int(shared), width, _stream()))
+    _check(_lib().ri_moe_act_weighted(_ptr(gate_up), gate_up.stride(0), _ptr(weights), _ptr(act), act.stride(0),
+                                      _dt(act), T, E, F, int(shared), width,
+                                      *_act_args(clip, weigh_input, shared_gate, T, "moe_swiglu_weighted"), _stream()))
 
 
 def moe_swiglu_routed(gate_up: torch.Tensor, logits: torch.Tensor, act: torch.Tensor, E: int, F: int, top: int,
                       renormalize: bool = False, score: str = "softmax", norm_eps: float = 0.0, scale: float = 1.0,
-                      shared: int = 0) -> None:
+                      shared: int = 0, clip: Optional[ClippedGate] = None, weigh_input: bool = False,
+                      shared_gate: Optional[torch.Tensor] = None) -> None:
     """``moe_route`` and ``moe_swiglu_weighted`` in one launch: the weights are made from the 32-bit
     ``logits [T, E]`` on the way and never stored."""
-    _dev(gate_up, logits, act)
+    _dev(gate_up, logits, act, shared_gate)
     _rows2d(gate_up, "gate_up")
     _rows2d(act, "act")
     _rows2d(logits, "logits")
     T, width = _moe_widths(gate_up, act, E, F, shared, "moe_swiglu_routed")
     if logits.dtype != torch.float32 or tuple(logits.shape) != (T, E):
         raise KernelError("moe_swiglu_routed: 32-bit logits [T, E] expected")
-    _check(_lib().ri_moe_swiglu_routed_as(_ptr(gate_up), gate_up.stride(0), _ptr(logits), logits.stride(0), _ptr(act),
-                                          act.stride(0), _dt(act), T, E, F, int(top), int(bool(renormalize)),
-                                          _score_kind(score), ctypes.c_float(norm_eps), ctypes.c_float(scale),
-                                          int(shared), width, _stream()))
+    _check(_lib().ri_moe_act_routed(_ptr(gate_up), gate_up.stride(0), _ptr(logits), logits.stride(0), _ptr(act),
+                                    act.stride(0), _dt(act), T, E, F, int(top), int(bool(renormalize)),
+                                    _score_kind(score), ctypes.c_float(norm_eps), ctypes.c_float(scale),
+                                    int(shared), width,
+                                    *_act_args(clip, weigh_input, shared_gate, T, "moe_swiglu_routed"), _stream()))
 
 
 # ---------------------------------------------------------------------------

@@ -15,7 +15,7 @@ from typing import Dict, List, Optional, Sequence
 
 import torch
 
-from ..parts.base import ParamSpec, Part, PositionEncoding, Runtime, join_name, narrow_tensors
+from ..parts.base import PagedKVNeed, ParamSpec, Part, PositionEncoding, Runtime, join_name, narrow_tensors
 from ..parts.block import Hidden
 from ..parts.embed import Embedding, LMHead
 
@@ -102,8 +102,12 @@ class DecoderModel(Part):
             need = self.layers[call.layer].cache_need()
             if need is None:
                 continue
-            if call.cache in needs and needs[call.cache] != need:
-                raise ValueError(f"cache {call.cache} is used with two different needs")
+            have = needs.get(call.cache)
+            if have is not None and have != need:
+                # layers may look at one cache through different windows or chunks: it keeps what any of them sees
+                if not (isinstance(have, PagedKVNeed) and isinstance(need, PagedKVNeed)):
+                    raise ValueError(f"cache {call.cache} is used with two different needs")
+                need = have.joined(need)
             needs[call.cache] = need
         return needs
 

@@ -154,7 +154,7 @@ class PagedAttention(Mixer):
 
 
 class WindowAttention(ProjectedPart, Mixer):
-    """Grouped softmax attention over the last ``window`` positions with key heads of size
+    """Grouped softmax attention over the last ``window`` positions (all without one) with key heads of size
     ``head_dim`` and value heads of size ``v_head_dim``.  ``pos_enc`` rotates the first
     ``pos_enc.rot_dim`` features of queries and keys; ``value_pos_enc`` (a rotation over all of
     ``v_head_dim``) is applied to every value before it is cached, by the value's position, and
@@ -176,7 +176,15 @@ class WindowAttention(ProjectedPart, Mixer):
     many positions of a sequence stay in sight, at their true positions; the cache never gives their pages back.
     ``sink``: a learned number a head (tensor ``sink``) whose exponential joins the softmax's denominator.
     ``sigmoid_weights``: no softmax; a visible key's weight is ``sigmoid(score + b_h)`` with a learned number a
-    head (tensor ``pb``), and the weights are not normalised over the keys."""
+    head (tensor ``pb``), and the weights are not normalised over the keys.
+
+    ``chunk``: positions are cut into chunks of this size, counted from a sequence's first position, and a query
+    sees the keys of its own chunk only; the cache gives the pages of finished chunks back.
+    ``difference`` (the design's constant ``d``): every query head makes two queries and every key head two keys of
+    ``head_dim`` (rows head by head: first map, second map) over one value.  With the two maps' outputs ``a``, ``b``
+    and one number a layer, ``lam = exp(lq1 . lk1) - exp(lq2 . lk2) + d`` (four tensors of ``head_dim``), a head's output
+    is ``(a - lam b)`` divided by its root mean square over the head (``difference_eps`` inside the root), times
+    ``1 - d``; ``a`` and ``b`` stay 32-bit.  The cached key row holds both maps' keys."""
 
     is_mixer = True
 
@@ -186,13 +194,19 @@ class WindowAttention(ProjectedPart, Mixer):
                  names: Optional[Dict[str, str]] = None, qk_norm_eps: Optional[float] = None,
                  q_temperature=None, own_kv: bool = True, interleaved: bool = False,
                  qk_unit_eps: Optional[float] = None, keep_first: int = 0, sink: bool = False,
-                 sigmoid_weights: bool = False):
+                 sigmoid_weights: bool = False, chunk: Optional[int] = None, difference: Optional[float] = None,
+                 difference_eps: float = 1e-5):
         if num_heads % num_kv_heads:
             raise ValueError(f"num_heads {num_heads} is not a multiple of num_kv_heads {num_kv_heads}")
         if sink and sigmoid_weights:
             raise ValueError("a sink belongs to a softmax: sigmoid weights take none")
-        if keep_first and not window:
+        if keep_first and not window and not chunk:
             keep_first = 0                       # without a window every position stays in sight anyway
+        self.chunk = int(chunk) if chunk else None
+        self.difference = float(difference) if difference is not None else None
+        self.difference_eps = float(difference_eps)
+        self.maps = 1 if difference is None else 2
+        self.lam = None
         self.interleaved = bool(interleaved)
         self.qk_unit_eps = float(qk_unit_eps) if qk_unit_eps else None
         self.keep_first = int(keep_first)
@@ -211,9 +225,12 @@ class WindowAttention(ProjectedPart, Mixer):
         self.window = int(window) if window else None
         self.pos_enc, self.value_pos_enc = pos_enc, value_pos_enc
         self.interleaved_values = bool(interleaved_values)
-        self.names = {"q": "q", "k": "k", "v": "v", "o": "o", "sink": "sink", "sigmoid_bias": "pb"}
+        self.names = {"q": "q", "k": "k", "v": "v", "o": "o", "sink": "sink", "sigmoid_bias": "pb",
+                      "lq1": "lq1", "lk1": "lk1", "lq2": "lq2", "lk2": "lk2"}
         if names:
             self.names.update(names)
+        if self.maps == 2 and (pos_enc is not None or value_pos_enc is not None or not self.by_head):
+            raise ValueError("the difference of two maps takes normed queries and keys without a rotation")
         if self.by_head and (self.interleaved or self.qk_unit_eps is not None):
             raise ValueError("the weighted norm of queries and keys goes without a rotation and without the unit norm")
 
@@ -226,17 +243,20 @@ class WindowAttention(ProjectedPart, Mixer):
 
     def in_projections(self):
         n = self.names
+        q, k = self.num_heads * self.maps * self.head_dim, self.num_kv_heads * self.maps * self.head_dim
         if not self.own_kv:
-            return [(n["q"], self.num_heads * self.head_dim)]
-        return [(n["q"], self.num_heads * self.head_dim), (n["k"], self.num_kv_heads * self.head_dim),
-                (n["v"], self.num_kv_heads * self.v_head_dim)]
+            return [(n["q"], q)]
+        return [(n["q"], q), (n["k"], k), (n["v"], self.num_kv_heads * self.v_head_dim)]
 
     def own_specs(self):
         n, specs = self.names, {}
         if self.has_sink:
-            specs[n["sink"]] = ParamSpec((self.num_heads,), mean=0.0, std=1.0)
+            specs[n["sink"]] = ParamSpec((self.num_heads * self.maps,), mean=0.0, std=1.0)
         if self.sigmoid_weights:
-            specs[n["sigmoid_bias"]] = ParamSpec((self.num_heads,), mean=-2.0, std=1.0)
+            specs[n["sigmoid_bias"]] = ParamSpec((self.num_heads * self.maps,), mean=-2.0, std=1.0)
+        if self.maps == 2:
+            for name in ("lq1", "lk1", "lq2", "lk2"):
+                specs[n[name]] = ParamSpec((self.head_dim,), mean=0.0, std=0.1)
         if self.qk_norm_eps is None:
             return specs
         specs[n["q"] + ".norm"] = ParamSpec((self.head_dim,), "norm")
@@ -248,7 +268,8 @@ class WindowAttention(ProjectedPart, Mixer):
         return (self.names["o"], self.num_heads * self.v_head_dim)
 
     def cache_need(self):
-        return PagedKVNeed(self.num_kv_heads, self.head_dim, self.window, self.v_head_dim, self.keep_first)
+        return PagedKVNeed(self.num_kv_heads, self.maps * self.head_dim, self.window, self.v_head_dim, self.keep_first,
+                           (self.chunk,) if self.chunk else ())
 
     def load_own(self, tensors, rt: Runtime) -> None:
         self.rt = rt
@@ -257,7 +278,10 @@ class WindowAttention(ProjectedPart, Mixer):
             self.sink = f32(self.names["sink"])
         if self.sigmoid_weights:
             self.sigmoid_bias = f32(self.names["sigmoid_bias"])
-        if not rt.ops.window_attention_supported(self.num_heads, self.num_kv_heads, self.head_dim, self.v_head_dim):
+        if self.maps == 2:
+            f64 = lambda name: tensors[self.names[name]].to(device="cpu", dtype=torch.float64)
+            self.lam = float(torch.exp(torch.sum(f64("lq1") * f64("lk1"))) - torch.exp(torch.sum(f64("lq2") * f64("lk2")))) + self.difference
+        if not rt.ops.window_attention_supported(self.num_heads, self.num_kv_heads, self.head_dim, self.v_head_dim, self.maps):
             raise ValueError(f"attention with {self.num_heads}/{self.num_kv_heads} heads of {self.head_dim} and "
                              f"{self.v_head_dim} features is beyond the window attention kernel")
         self.q_norm_weight = self.k_norm_weight = None
@@ -276,9 +300,9 @@ class WindowAttention(ProjectedPart, Mixer):
             ops.head_norm_kv_write(q, k, v, self.num_heads, self.num_kv_heads, self.head_dim, self.v_head_dim,
                                    self.q_norm_weight, self.k_norm_weight, self.qk_norm_eps or 1.0, ctx.positions,
                                    ctx.row_of_token, cache.k, cache.v, table, cache.page_size, write_kv=write,
-                                   norm=self.qk_norm_eps is not None, temp_coef=coef, temp_every=every)
+                                   norm=self.qk_norm_eps is not None, temp_coef=coef, temp_every=every, maps=self.maps)
             ops.window_attention(q, act, self.num_heads, self.num_kv_heads, self.head_dim, self.v_head_dim, cache.k, cache.v,
-                                 table, cache.page_size, ctx, self.scale, self.window or 0, None, False)
+                                 table, cache.page_size, ctx, self.scale, self.window or 0, None, False, **self._weights_how())
             return
         rotary = self.pos_enc.rotary() if self.pos_enc is not None else None
         vrot = self.value_pos_enc.rotary()[:2] if self.value_pos_enc is not None else None
@@ -288,15 +312,24 @@ class WindowAttention(ProjectedPart, Mixer):
         ops.rotate_kv_write(q, k, v, self.num_heads, self.num_kv_heads, self.head_dim, self.v_head_dim, rotary, vrot,
                             ctx.positions, ctx.row_of_token, cache.k, cache.v, table, cache.page_size,
                             write_kv=write, interleaved_values=self.interleaved_values, **extra)
-        extra = {}
-        if self.sink is not None:
-            extra["sink"] = self.sink
-        if self.keep_first:
-            extra["keep_first"] = self.keep_first
-        if self.sigmoid_bias is not None:
-            extra["sigmoid_bias"] = self.sigmoid_bias
         ops.window_attention(q, act, self.num_heads, self.num_kv_heads, self.head_dim, self.v_head_dim, cache.k, cache.v,
-                             table, cache.page_size, ctx, self.scale, self.window or 0, vrot, self.interleaved_values, **extra)
+                             table, cache.page_size, ctx, self.scale, self.window or 0, vrot, self.interleaved_values,
+                             **self._weights_how())
+
+    def _weights_how(self):
+        """What the attention kernels are told beside the sizes, the scale and the window."""
+        how = {}
+        if self.sink is not None:
+            how["sink"] = self.sink
+        if self.keep_first:
+            how["keep_first"] = self.keep_first
+        if self.sigmoid_bias is not None:
+            how["sigmoid_bias"] = self.sigmoid_bias
+        if self.chunk:
+            how["chunk"] = self.chunk
+        if self.maps == 2:
+            how["difference"] = (self.lam, 1.0 - self.difference, self.difference_eps)
+        return how
 
 
 class LatentAttention(ProjectedPart, Mixer):

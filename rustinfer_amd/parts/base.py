@@ -65,17 +65,41 @@ class ParamSpec:
 
 @dataclass(frozen=True)
 class PagedKVNeed:
-    """Keys and values of every position (or of the last ``window`` positions).  ``v_head_dim``:
-    the size of a value head where it differs from a key head's."""
+    """Keys and values of every position, of the last ``window`` positions, or of the query's own chunk of
+    positions (counted from the request's first).  ``v_head_dim``: the size of a value head where it differs
+    from a key head's."""
     num_kv_heads: int
     head_dim: int
     window: Optional[int] = None
     v_head_dim: Optional[int] = None
     keep_first: int = 0       # with a window: the first so many positions stay readable, their pages are never given back
+    # sizes of the chunks in which a position is read (several where layers of different chunks read one cache)
+    chunks: Tuple[int, ...] = ()
 
     @property
     def value_dim(self) -> int:
         return self.head_dim if self.v_head_dim is None else self.v_head_dim
+
+    @property
+    def bounded(self) -> bool:
+        """Whether positions go out of sight (and their pages can be given back)."""
+        return self.window is not None or bool(self.chunks)
+
+    def first_position(self, next_pos: int) -> int:
+        """The lowest position a query at ``next_pos`` or later reads (kept first positions aside)."""
+        reach = [next_pos - self.window + 1] if self.window is not None else []
+        reach += [next_pos - next_pos % c for c in self.chunks]
+        return max(0, min(reach)) if reach else 0
+
+    def joined(self, other: "PagedKVNeed") -> "PagedKVNeed":
+        """The need of a cache that layers with both needs read: everything either of them may see."""
+        if (self.num_kv_heads, self.head_dim, self.value_dim) != (other.num_kv_heads, other.head_dim, other.value_dim):
+            raise ValueError(f"one cache cannot hold heads of {self} and {other}")
+        if not (self.bounded and other.bounded):
+            return PagedKVNeed(self.num_kv_heads, self.head_dim, None, self.v_head_dim)
+        windows = [w for w in (self.window, other.window) if w is not None]
+        return PagedKVNeed(self.num_kv_heads, self.head_dim, max(windows, default=None), self.v_head_dim,
+                           max(self.keep_first, other.keep_first), tuple(sorted(set(self.chunks) | set(other.chunks))))
 
 
 @dataclass(frozen=True)

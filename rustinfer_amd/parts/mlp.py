@@ -157,7 +157,11 @@ class MoEFeedForward(FeedForward):
     chosen scores are divided by their sum + ``norm_eps``; ``scale`` multiplies the weights.
     ``shared_size`` > 0: one more gated feed-forward of that width (tensors ``shared.gate|up|down``) that every
     token uses with weight 1: its gate and up rows are stacked under the experts' and its down columns beside
-    theirs, so it rides in the same two products.
+    theirs, so it rides in the same two products.  ``shared_gate``: the shared expert's output is multiplied by the
+    sigmoid of one more logit a token (tensor ``shared.sg``); its row stands under the router's in the same product.
+    ``limit``: every expert's activation is the clipped one, ``g' sigmoid(slope g') (u' + shift)`` with
+    ``g' = min(g, limit)`` and ``u' = clamp(u, -limit, limit)`` (``shared_limit``: the shared expert's limit).
+    ``weigh_input``: an expert runs on its token's row multiplied by the weight, instead of its output being multiplied.
     Tensor names: ``router``, ``e<i>.gate``, ``e<i>.up``, ``e<i>.down``."""
 
     # up to this many tokens in a step every block of the activation kernel makes its token's weights
@@ -166,7 +170,9 @@ class MoEFeedForward(FeedForward):
     ROUTE_ON_THE_WAY_ROWS = 64
 
     def __init__(self, hidden_size: int, expert_size: int, experts: int, top: int, renormalize: bool = False,
-                 score: str = "softmax", norm_eps: float = 0.0, scale: float = 1.0, shared_size: int = 0):
+                 score: str = "softmax", norm_eps: float = 0.0, scale: float = 1.0, shared_size: int = 0,
+                 shared_gate: bool = False, limit: Optional[float] = None, shared_limit: Optional[float] = None,
+                 slope: float = 1.702, shift: float = 1.0, weigh_input: bool = False):
         if not (0 < top <= experts):
             raise ValueError(f"top {top} of {experts} experts")
         if score not in ("softmax", "sigmoid"):
@@ -174,10 +180,18 @@ class MoEFeedForward(FeedForward):
         self.hidden_size, self.expert_size = int(hidden_size), int(expert_size)
         self.experts, self.top, self.renormalize = int(experts), int(top), bool(renormalize)
         self.score, self.norm_eps, self.scale, self.shared_size = score, float(norm_eps), float(scale), int(shared_size)
+        if shared_gate and not shared_size:
+            raise ValueError("a shared expert's gate needs a shared expert")
+        self.shared_gate, self.weigh_input = bool(shared_gate), bool(weigh_input)
+        self.limit = float(limit) if limit is not None else None
+        self.shared_limit = float(shared_limit) if shared_limit is not None else self.limit
+        self.slope, self.shift = float(slope), float(shift)
+        self.clip = None
         self.plain = score == "softmax" and self.scale == 1.0 and self.norm_eps == 0.0 and self.shared_size == 0
         # columns of the activations: the experts', the shared expert's, zeros up to a multiple of eight
         self.act_width = (self.experts * self.expert_size + self.shared_size + 7) // 8 * 8
-        self.router = Linear(self.hidden_size, self.experts)
+        self.logits_width = self.experts + int(self.shared_gate)
+        self.router = Linear(self.hidden_size, self.logits_width)
         self.gate_up = Linear(self.hidden_size, 2 * self.experts * self.expert_size + 2 * self.shared_size)
         self.down = Linear(self.act_width, self.hidden_size)
 
@@ -189,12 +203,19 @@ class MoEFeedForward(FeedForward):
         if self.shared_size:
             s = self.shared_size
             specs["shared.gate"], specs["shared.up"], specs["shared.down"] = ParamSpec((s, h)), ParamSpec((s, h)), ParamSpec((h, s))
+        if self.shared_gate:
+            specs["shared.sg"] = ParamSpec((1, h))
         return specs
 
     def load(self, tensors, rt: Runtime) -> None:
         self.rt = rt
         to = lambda name: tensors[name].to(device=rt.device, dtype=rt.dtype)
-        self.router.set_weight(to("router"), rt, tile=False)
+        router = to("router")
+        if self.shared_gate:
+            router = torch.cat([router, to("shared.sg")], dim=0)
+        self.router.set_weight(router, rt, tile=False)
+        if self.limit is not None:
+            self.clip = rt.ops.ClippedGate(self.limit, self.shared_limit, self.slope, self.shift)
         rows = [to(f"e{e}.{n}") for e in range(self.experts) for n in ("gate", "up")]
         cols = [to(f"e{e}.down") for e in range(self.experts)]
         if self.shared_size:
@@ -209,13 +230,20 @@ class MoEFeedForward(FeedForward):
     def forward(self, ctx, normed) -> torch.Tensor:
         ops, ws = self.rt.ops, ctx.workspace
         T, E, F = normed.shape[0], self.experts, self.expert_size
-        logits = ws.get("moe.logits", T, E, torch.float32)
+        logits = ws.get("moe.logits", T, self.logits_width, torch.float32)
         self.router.forward(normed, logits)
         gate_up = ws.get("moe.gate_up", T, 2 * E * F + 2 * self.shared_size, self.rt.dtype)
         self.gate_up.forward(normed, gate_up)
         act = ws.get("moe.act", T, self.act_width, self.rt.dtype)
         how = {} if self.plain else {"score": self.score, "norm_eps": self.norm_eps, "scale": self.scale}
         shared = {} if self.plain else {"shared": self.shared_size}
+        if self.shared_gate:
+            shared["shared_gate"] = logits[:, E]
+            logits = logits[:, :E]
+        if self.clip is not None:
+            shared["clip"] = self.clip
+        if self.weigh_input:
+            shared["weigh_input"] = True
         if T <= self.ROUTE_ON_THE_WAY_ROWS:
             ops.moe_swiglu_routed(gate_up, logits, act, E, F, self.top, self.renormalize, **how, **shared)
         else:
