@@ -609,14 +609,46 @@ class DebuzenBench(TedelixBench):
         self.weight_bytes = el * self.params
 
 
+# Zotonex at the layer sizes of the Llama shapes: the same width and number of layers; a head of two maps counts as two
+# of the shape's heads (queries and keys of the shape's head size a map, values twice as wide), so the projections and the
+# cache are the shape's; every other layer reads the keys and values of the layer before it; chunks of 8,192 positions
+# (longer than the requests here, so that they read all their keys as Belorax's do); in every layer Belorax's eight experts
+# of a quarter of the shape's feed-forward width, two a token, and a gated shared one of that width.
+def zotonex_config(shape_name, layers=0, chunk=8192):
+    s = SHAPES[shape_name]
+    H, G, hd, W, ff = s["num_attention_heads"], s["num_key_value_heads"], s["head_dim"], s["hidden_size"], s["intermediate_size"]
+    out = []
+    for i in range(layers or s["num_hidden_layers"]):
+        mixer = dict(heads=H // 2, kv_heads=max(G // 2, 1), dim=hd, vdim=2 * hd, scale=hd ** -0.5, diff=0.3, mask=dict(size=chunk))
+        if i % 2 == 1:
+            mixer["kv_from"] = i - 1
+        mlp = dict(kind="moe", expert=dict(ff=ff // 4, limit=7.0), router=dict(experts=8, top=2), shared=dict(ff=ff // 4, limit=7.0))
+        out.append(dict(type="attention", mixer=mixer, mlp=mlp))
+    return dict(architecture="Zotonex", vocab=s["vocab_size"], width=W, norm=dict(eps=1e-6), embedding=dict(scale=1.0), logit_scale=0.5, layers=out)
+
+
+class ZotonexBench(TedelixBench):
+    """The same measurements on a Zotonex model of a Llama shape's sizes."""
+
+    def design_config(self, shape_name, args):
+        self.window = 1 << 30                         # the chunk is longer than the requests: they read all their keys
+        return zotonex_config(shape_name, args.layers)
+
+    def account(self, cfg, el):
+        self.state_bytes = self.scan_flops_per_token = 0
+        self.window_kv_bytes = sum(l.mixer.kv_heads * (2 * l.mixer.dim + l.mixer.vdim) * el for l in cfg.layers)    # a borrowed cache is read again
+        self.attn_flops_per_key = sum(2.0 * 2 * l.mixer.heads * (l.mixer.dim + l.mixer.vdim) for l in cfg.layers)
+
+
 DESIGNS = {"tedelix": (TedelixBench, "llama", TEDELIX_PATTERN), "belorax": (BeloraxBench, "tedelix", BELORAX_PATTERN),
-           "pilavik": (PilavikBench, "belorax", PILAVIK_PATTERN), "debuzen": (DebuzenBench, "pilavik", DEBUZEN_PATTERN)}
+           "pilavik": (PilavikBench, "belorax", PILAVIK_PATTERN), "debuzen": (DebuzenBench, "pilavik", DEBUZEN_PATTERN),
+           "zotonex": (ZotonexBench, "belorax", ("attention", "attention on a borrowed cache"))}
 
 
 def design_record(args, peaks):
-    """``--design tedelix|belorax|pilavik|debuzen``: decode at the main batch and prefill of 2,048 tokens for
+    """``--design tedelix|belorax|pilavik|debuzen|zotonex``: decode at the main batch and prefill of 2,048 tokens for
     models of that design at the sizes of ``--design-shapes``, each beside the closest other design at the same
-    sizes (Tedelix beside Llama, Belorax beside Tedelix, Pilavik beside Belorax, Debuzen beside Pilavik)."""
+    sizes (Tedelix beside Llama, Belorax beside Tedelix, Pilavik beside Belorax, Debuzen beside Pilavik, Zotonex beside Belorax)."""
     design_cls, beside, pattern = DESIGNS[args.design]
     others = {"llama": Bench, "tedelix": TedelixBench, "belorax": BeloraxBench, "pilavik": PilavikBench}
     out = {"metric": "decode tok/s at batch %d and prefill tok/s at 2,048 tokens: %s beside %s at equal layer sizes" % (args.batch, args.design, beside),
@@ -719,10 +751,10 @@ def main() -> int:
                     help="only time the sampling kernels on 1, 8 and 64 rows of the shape's vocabulary")
     ap.add_argument("--no-gemm-tune", action="store_true",
                     help="keep the GEMM library's own choice of kernel for the prompt's products")
-    ap.add_argument("--design", default="llama", choices=["llama", "tedelix", "belorax", "pilavik", "debuzen"],
-                    help="tedelix, belorax, pilavik, debuzen: only decode and prefill of models of that design at the sizes of "
+    ap.add_argument("--design", default="llama", choices=["llama", "tedelix", "belorax", "pilavik", "debuzen", "zotonex"],
+                    help="tedelix, belorax, pilavik, debuzen, zotonex: only decode and prefill of models of that design at the sizes of "
                          "--design-shapes, each beside the closest other design at the same sizes (Tedelix beside Llama, "
-                         "Belorax beside Tedelix, Pilavik beside Belorax; the default workload is not run)")
+                         "Belorax beside Tedelix, Pilavik beside Belorax, Debuzen beside Pilavik, Zotonex beside Belorax; the default workload is not run)")
     ap.add_argument("--design-shapes", default="1b,3b", help="shapes for --design other than llama, with commas between them")
     args = ap.parse_args()
     if args.gpus != 1:

@@ -136,13 +136,14 @@ def expert(h, w, limit: float):
 
 
 def routed_ff(h, w, mlp, gaps=None):
-    """``gaps`` (a list) receives, for every row, how far the last chosen expert's score lies above the
-    first one left out, relative to it (infinite where all experts are chosen)."""
+    """``gaps`` (a list) receives, for every row, how far the last chosen expert's logit lies above the
+    first one left out (infinite where all experts are chosen)."""
     E, top = mlp["router"]["experts"], mlp["router"]["top"]
-    s = sigmoid(h @ w["router"].T)
+    z = h @ w["router"].T
+    s = sigmoid(z)
     if gaps is not None:
-        ranked = -np.sort(-s, axis=1)
-        gaps.append((ranked[:, top - 1] - ranked[:, top]) / ranked[:, top - 1] if top < E else np.full(h.shape[0], np.inf))
+        ranked = -np.sort(-z, axis=1)
+        gaps.append(ranked[:, top - 1] - ranked[:, top] if top < E else np.full(h.shape[0], np.inf))
     out = np.zeros((h.shape[0], w["e0.down"].shape[0]))
     for t in range(h.shape[0]):
         for e in np.argsort(-s[t], kind="stable")[:top]:
