@@ -998,6 +998,9 @@ def rotate_kv_write(q: torch.Tensor, k: Optional[torch.Tensor], v: Optional[torc
         int(bool(write_kv)), ctypes.c_float(unit_eps), _stream()))
 
 
+# bfloat16 attention without turned values, kept first positions and sigmoid weights, on pages of a multiple of 16, takes the
+# kernels of attention_parts.hip (False: the ones below, for comparison)
+WINDOW_ATTENTION_PARTS = True
 WINDOW_ATTENTION_MFMA = True     # steps with prompt portions take the matrix-instruction kernel (False: the FMA one, for comparison)
 
 
@@ -1047,6 +1050,22 @@ def window_attention(q: torch.Tensor, out: torch.Tensor, H: int, Hkv: int, dk: i
     _i32(ctx.kv_lens, "kv_lens", ctx.num_rows)
     vcos, vsin, vrows = _rot_tables(value_rotary, dv, "window_attention (values)")
     lib = _lib()
+    single = int(ctx.max_q_len == 1 and T <= ctx.num_rows)
+    if WINDOW_ATTENTION_PARTS and q.dtype == torch.bfloat16 and value_rotary is None and keep_first == 0 and sigmoid_bias is None \
+            and scale > 0 and q.stride(0) % 8 == 0 and q.data_ptr() % 16 == 0 \
+            and lib.ri_attention_parts_supported(H, Hkv, dk, dv, maps, page):
+        # both products on the bfloat16 matrix instructions, the weights as three bfloat16 parts
+        ws, need = None, 0
+        if single:
+            lib.ri_attention_parts_workspace.restype = ctypes.c_size_t
+            need = lib.ri_attention_parts_workspace(T, H, dv, maps, int(window), int(chunk), int(ctx.max_kv_len))
+            ws = ctx.workspace.get("attn.window_partials", need, 1, torch.float32)
+        _check(lib.ri_attention_parts(
+            _ptr(q), q.stride(0), _ptr(out), out.stride(0), _ptr(k_cache), _ptr(v_cache), k_cache.shape[0], page,
+            H, Hkv, dk, dv, _ptr(block_table), block_table.shape[1], _ptr(ctx.cu_q), _ptr(ctx.q_start), _ptr(ctx.kv_lens),
+            ctx.num_rows, T, ctypes.c_float(scale), int(window), int(chunk), maps, lam, gain, diff_eps, _ptr(sink),
+            single, int(ctx.max_kv_len), _ptr(ws), ctypes.c_size_t(need), _stream()))
+        return
     if ctx.max_q_len > 1 and WINDOW_ATTENTION_MFMA and lib.ri_attention_window_mfma_supported(H, Hkv, dk, dv, maps):
         # steps with prompt portions: both products on the 32-bit matrix instructions
         _check(lib.ri_attention_window_mfma(
@@ -1056,7 +1075,7 @@ def window_attention(q: torch.Tensor, out: torch.Tensor, H: int, Hkv: int, dk: i
             keep_first, _ptr(sigmoid_bias), int(chunk), maps, lam, gain, diff_eps, _stream()))
         return
     # a step of single tokens divides each row's keys between blocks, through a workspace
-    single, ws, need = int(ctx.max_q_len == 1 and T <= ctx.num_rows), None, 0
+    ws, need = None, 0
     if single:
         lib.ri_attention_window_workspace.restype = ctypes.c_size_t
         need = lib.ri_attention_window_workspace(T, H, dv, int(window), int(chunk), int(ctx.max_kv_len), keep_first, maps)

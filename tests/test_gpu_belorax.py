@@ -239,12 +239,13 @@ class OnePart:
         return {0: need} if need is not None else {}
 
 
-def run_part(part, pos_encs, dtype, x, cuts, page=8, batch_with=None):
+def run_part(part, pos_encs, dtype, x, cuts, page=8, batch_with=None, num_pages=160, max_len=640):
     """The part's output [T, hidden] for one sequence ``x [T, hidden]`` fed in portions of ``cuts``.
     ``batch_with``: rows of a second request that shares every step (its output is dropped)."""
     from rustinfer_amd.engine import Engine, StepEntry, make_runtime
     rt = make_runtime(dtype, DEV)
-    eng = Engine(OnePart(part, pos_encs), rt, page_size=page, num_pages=160, max_requests=3, max_model_len=640)
+    eng = Engine(OnePart(part, pos_encs), rt, page_size=page, num_pages=num_pages, max_requests=3, max_model_len=max_len,
+                 max_batch_tokens=max(8192, max_len))
     outs, pos, other = [], 0, 0
     for n in cuts:
         entries, rows = [StepEntry("a", [0] * n, [])], [x[pos:pos + n]]
@@ -291,13 +292,15 @@ def some_rows(T, d, seed):
     return torch.randn(T, d, generator=torch.Generator().manual_seed(seed)).to(torch.bfloat16).float()
 
 
-@pytest.fixture(params=["matrix", "fma"])
+@pytest.fixture(params=["parts", "matrix", "fma"])
 def portion_kernel(request):
-    """Steps with prompt portions on the matrix-instruction kernel (the default) and on the FMA one."""
+    """Attention on the kernels an engine chooses by default (bfloat16: the bfloat16 matrix instructions with weights in
+    parts, where they take the sizes), on the 32-bit matrix instructions, and on the FMA kernel."""
     from rustinfer_amd.kernels import ops
-    keep, ops.WINDOW_ATTENTION_MFMA = ops.WINDOW_ATTENTION_MFMA, request.param == "matrix"
+    keep = ops.WINDOW_ATTENTION_PARTS, ops.WINDOW_ATTENTION_MFMA
+    ops.WINDOW_ATTENTION_PARTS, ops.WINDOW_ATTENTION_MFMA = request.param == "parts", request.param != "fma"
     yield request.param
-    ops.WINDOW_ATTENTION_MFMA = keep
+    ops.WINDOW_ATTENTION_PARTS, ops.WINDOW_ATTENTION_MFMA = keep
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
@@ -315,7 +318,7 @@ def test_normed_attention_alone(dtype, H, G, dk, dv, scale, coef, every, portion
     m = dict(heads=H, kv_heads=G, dim=dk, vdim=dv, scale=scale, q_temp=dict(coef=coef, every=every or 1 << 30))
     xs = x.double().numpy()
     ref = P.qknorm_attention(xs, w, m, 1e-5, P.attention_keys_values(xs, w, m, 1e-5))
-    assert rel(run_part(part, [], dtype, x, CUTS), ref) < PART_TOL[dtype]
+    assert rel(run_part(part, [], dtype, x, CUTS, page=16 if portion_kernel == "parts" else 8), ref) < PART_TOL[dtype]
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
@@ -338,7 +341,7 @@ def test_latent_attention_alone(dtype, H, d, r, dv, R, dims, scaling, portion_ke
         rot["scaling"] = scaling
     m = dict(heads=H, dim=d, rot_dim=r, vdim=dv, kv_rank=R, scale=0.3 / math.sqrt(d + r), rot=rot)
     ref = P.latent_attention(x.double().numpy(), w, m, 1e-5)
-    assert rel(run_part(part, [pe], dtype, x, CUTS), ref) < PART_TOL[dtype]
+    assert rel(run_part(part, [pe], dtype, x, CUTS, page=16 if portion_kernel == "parts" else 8), ref) < PART_TOL[dtype]
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])

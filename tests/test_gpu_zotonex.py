@@ -186,16 +186,61 @@ def plain_attention(xs, w, m, eps=1e-5):
 @pytest.mark.parametrize("H,G,dk,dv,scale,size,diff", [
     (4, 2, 16, 24, 0.3, 23, 0.3), (3, 3, 40, 36, 0.2, 64, 0.0), (8, 1, 32, 16, 0.18, 16, 0.8), (2, 2, 128, 128, 0.09, 100, 0.5),
     (5, 5, 72, 200, 0.12, 7, 0.1), (6, 1, 24, 40, 0.2, 150, 0.6), (2, 1, 256, 256, 0.06, 40, 0.4), (1, 1, 6, 2, 0.5, 1, 0.2),
-    (16, 1, 8, 12, 0.35, 48, 0.45), (6, 2, 64, 128, 0.12, None, 0.3), (12, 4, 20, 72, 0.25, 33, 0.9), (3, 1, 10, 100, 0.3, 5, 0.35)])
+    (16, 1, 8, 12, 0.35, 48, 0.45), (6, 2, 64, 128, 0.12, None, 0.3), (12, 4, 24, 72, 0.25, 33, 0.9), (3, 1, 10, 100, 0.3, 5, 0.35),
+    (10, 1, 16, 64, 0.3, 80, 0.25), (4, 4, 104, 256, 0.1, 33, 0.3), (9, 3, 40, 56, 0.2, None, 0.15)])
 def test_difference_attention_alone(dtype, H, G, dk, dv, scale, size, diff, portion_kernel):
     d, m = 48, att(H, G, dk, dv, scale, size, diff)
     part = attention_part(d, m)
     w = load_part(part, H * dk + dv, dtype, scale=2.0)
     x = some_rows(sum(CUTS), d, 5)
     ref = plain_attention(x.double().numpy(), w, m)
-    assert rel(run_part(part, [], dtype, x, CUTS), ref) < PART_TOL[dtype]
+    page = 16 if portion_kernel == "parts" else 8
+    assert rel(run_part(part, [], dtype, x, CUTS, page=page), ref) < PART_TOL[dtype]
     other = some_rows(60, d, 8)
-    assert rel(run_part(part, [], dtype, x, CUTS, batch_with=other), ref) < PART_TOL[dtype]     # another request beside it
+    assert rel(run_part(part, [], dtype, x, CUTS, page=page, batch_with=other), ref) < PART_TOL[dtype]     # another request beside it
+
+
+@pytest.mark.parametrize("size", [None, 4100])
+def test_thousands_of_keys(size):
+    """A prompt of 4,300 tokens and single tokens behind it: more stretches of keys than a row may leave partial
+    results of, so that a wave of the single-token kernel takes several; every query has a favourite far back."""
+    T, d = 4330, 32
+    m = att(4, 2, 16, 24, 1.2, size, 0.3)
+    part = attention_part(d, m)
+    w = load_part(part, 3, "bfloat16", scale=2.0)
+    x = some_rows(T, d, 11)
+    ref = plain_attention(x.double().numpy(), w, m)
+    cuts = [2048, 2200, 52] + [1] * 30
+    got = run_part(part, [], "bfloat16", x, cuts, page=16, num_pages=300, max_len=4400)
+    assert rel(got[:4100], ref[:4100]) < PART_TOL["bfloat16"] and rel(got[4100:], ref[4100:]) < PART_TOL["bfloat16"]
+
+
+def test_weights_keep_their_32_bits(monkeypatch):
+    """The bfloat16 kernels against the 32-bit ones on the same bfloat16 queries, keys and values: far closer than
+    weights rounded to bfloat16 would be (4e-3), in portions and in single tokens."""
+    from rustinfer_amd.kernels import ops
+    d, m = 48, att(4, 2, 64, 64, 0.12, 100, 0.3)
+    x = some_rows(sum(CUTS), d, 5)
+    outs = []
+    for parts in (True, False):
+        monkeypatch.setattr(ops, "WINDOW_ATTENTION_PARTS", parts)
+        keep = []
+        real = ops.window_attention
+
+        def both(q, out, *args, **kw):
+            wide = torch.empty(out.shape, device=out.device, dtype=torch.bfloat16)
+            real(q, wide, *args, **kw)
+            out.copy_(wide)
+            keep.append(wide.double().cpu().numpy())
+        monkeypatch.setattr(ops, "window_attention", both)
+        part = attention_part(d, m)
+        load_part(part, 5, "bfloat16", scale=2.0)
+        run_part(part, [], "bfloat16", x, CUTS, page=16)
+        monkeypatch.setattr(ops, "window_attention", real)
+        outs.append(np.concatenate(keep))
+    diff = np.abs(outs[0] - outs[1])
+    # results that round to neighbouring bfloat16 numbers now and then, almost never further apart
+    assert (diff > 0).mean() < 0.02 and diff.max() < 2.0 ** -7 * np.abs(outs[1]).max()
 
 
 @pytest.mark.parametrize("mistake", ["maps swapped", "values of the second map", "no second map", "no factor", "one less in the exponent"])
