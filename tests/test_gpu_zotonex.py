@@ -591,10 +591,11 @@ def draw_config(rng):
                 norm=dict(eps=pick([1e-5, 1e-6])), embedding=dict(scale=pick([1.0, 4.0, 12.0])), logit_scale=pick([0.1, 1.0, 3.0]), layers=layers)
 
 
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("seed", [11, 12, 13, 14, 15, 16, 17, 18])
-def test_configurations_drawn_at_random(seed, tmp_path):
-    """In 32-bit, where rounding hides nothing: last tokens alone, portions, and a mixed schedule on a pool
-    that is too small for all requests at once, against the plain implementation."""
+def test_configurations_drawn_at_random(seed, dtype, tmp_path):
+    """Last tokens alone, portions, and a mixed schedule on a pool that is too small for all requests at once, against
+    the plain implementation; 32-bit is the sharp test, bfloat16 goes through the kernels that serving uses."""
     from rustinfer_amd.engine import build_engine
     from rustinfer_amd.weights import write_safetensors
     cfg = draw_config(np.random.default_rng(seed))
@@ -605,9 +606,9 @@ def test_configurations_drawn_at_random(seed, tmp_path):
     reqs = random_requests(cfg["vocab"], (150, 3, 290, 40, 1, 77), seed)
     logits = plain_rows(cfg, w, reqs)
     max_tokens = 2 * 320 + 64
-    eng = build_engine(str(tmp_path), dtype="float32", device=DEV, page_size=16, num_pages=max_tokens // 16, max_requests=4,
+    eng = build_engine(str(tmp_path), dtype=dtype, device=DEV, page_size=16, num_pages=max_tokens // 16, max_requests=4,
                        max_model_len=max_tokens, max_batch_tokens=2048)
     for label, steps in (("last tokens alone", cut_tail_single(reqs, tail=40)), ("portions", cut_portions(reqs, seed=seed)),
                          ("mixed", cut_mixed(reqs, max_tokens, seed=seed, max_live=4, tail=6))):
-        check_rows(steps, run_steps(eng, steps), logits, "float32", f"{json.dumps(cfg)} {label}")
+        check_rows(steps, run_steps(eng, steps), logits, dtype, f"{json.dumps(cfg)} {label}")
         assert not eng.cache.live_requests()
