@@ -1365,3 +1365,230 @@ class ZotonexConfig(ModelConfig):
         if self.eos_token_ids:
             d["eos_token_id"] = list(self.eos_token_ids)
         return d
+
+
+# ---------------------------------------------------------------------------
+# Sibodra: several residual streams, soft-capped attention with an unlearned sink and a gate a head, attention through
+# latents of queries and of keys and values, experts without a gate
+# ---------------------------------------------------------------------------
+def _llama3_rot_of(m: Dict[str, Any], where: str):
+    """(base, dims, scaling) of a mixer's 'rot' object whose scaling, if there is one, is llama3's band by band."""
+    rot = _obj(m, "rot", where)
+    w = where + ".rot"
+    base, dims, sc = _require(rot, "base", float, w), _require(rot, "dims", int, w), rot.get("scaling")
+    if not base > 0 or dims <= 0 or dims % 2:
+        raise ConfigError(f"{w}: base must be > 0 and dims even and > 0")
+    if sc is None:
+        return base, dims, None
+    if not isinstance(sc, dict):
+        raise ConfigError(f"{w}: 'scaling' must be an object or null")
+    w += ".scaling"
+    s = RopeScaling("llama3", _require(sc, "factor", float, w), _require(sc, "low", float, w), _require(sc, "high", float, w),
+                    _require(sc, "original", float, w))
+    if not (s.factor > 0 and s.original_max_position_embeddings > 0 and 0 < s.low_freq_factor < s.high_freq_factor):
+        raise ConfigError(f"{w}: factor, low and original must be > 0 and high must exceed low")
+    return base, dims, s
+
+
+def _llama3_rot_dict(base, dims, scaling: Optional[RopeScaling]) -> Dict[str, Any]:
+    d: Dict[str, Any] = {"base": base, "dims": dims}
+    if scaling is not None:
+        d["scaling"] = {"factor": scaling.factor, "low": scaling.low_freq_factor, "high": scaling.high_freq_factor,
+                        "original": scaling.original_max_position_embeddings}
+    return d
+
+
+@dataclass(frozen=True)
+class CappedAttentionSpec:
+    """Mixer ``attention``: normed and rotated queries and keys, scores soft-capped at ``softcap`` (None: not), a sink of
+    score 0 in the softmax, one output gate a head."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    softcap: Optional[float]
+    rot_base: float
+    rot_dims: int
+    rot_scaling: Optional[RopeScaling] = None
+    kind: str = "attention"
+
+    @staticmethod
+    def from_dict(m: Dict[str, Any], where: str) -> "CappedAttentionSpec":
+        base, dims, scaling = _llama3_rot_of(m, where)
+        cap = m.get("softcap")
+        s = CappedAttentionSpec(
+            heads=_require(m, "heads", int, where), kv_heads=_require(m, "kv_heads", int, where),
+            dim=_require(m, "dim", int, where), vdim=_require(m, "vdim", int, where), scale=_require(m, "scale", float, where),
+            softcap=_typed(cap, "softcap", float, where) if cap is not None else None,
+            rot_base=base, rot_dims=dims, rot_scaling=scaling)
+        if min(s.heads, s.kv_heads, s.dim, s.vdim) <= 0 or s.heads % s.kv_heads:
+            raise ConfigError(f"{where}: heads, kv_heads, dim and vdim must be > 0 and heads a multiple of kv_heads")
+        if s.rot_dims > s.dim:
+            raise ConfigError(f"{where}: rot.dims {s.rot_dims} exceeds dim {s.dim}")
+        if s.softcap is not None and not s.softcap > 0:
+            raise ConfigError(f"{where}: softcap must be > 0")
+        if max(s.dim, s.vdim) > MAX_HEAD_DIM or s.heads // s.kv_heads > 32:
+            raise ConfigError(f"{where}: heads of more than {MAX_HEAD_DIM} features or more than 32 query heads a key/value "
+                              f"head are beyond the attention kernels")
+        return s
+
+    def to_dict(self) -> Dict[str, Any]:
+        d = {"heads": self.heads, "kv_heads": self.kv_heads, "dim": self.dim, "vdim": self.vdim, "scale": self.scale,
+             "rot": _llama3_rot_dict(self.rot_base, self.rot_dims, self.rot_scaling)}
+        if self.softcap is not None:
+            d["softcap"] = self.softcap
+        return d
+
+
+@dataclass(frozen=True)
+class QueryLatentAttentionSpec:
+    """Mixer ``latent_attention``: queries come from a normed latent of ``q_rank`` features, keys and values from another
+    of ``kv_rank``, beside one rotated key part of ``rot_dim`` features for all heads; an output gate a feature."""
+    heads: int
+    dim: int                 # unrotated query/key features a head
+    rot_dim: int             # rotated query/key features a head
+    vdim: int
+    q_rank: int
+    kv_rank: int
+    scale: float
+    rot_base: float
+    rot_dims: int
+    rot_scaling: Optional[RopeScaling] = None
+    kind: str = "latent_attention"
+
+    @staticmethod
+    def from_dict(m: Dict[str, Any], where: str) -> "QueryLatentAttentionSpec":
+        base, dims, scaling = _llama3_rot_of(m, where)
+        s = QueryLatentAttentionSpec(
+            heads=_require(m, "heads", int, where), dim=_require(m, "dim", int, where),
+            rot_dim=_require(m, "rot_dim", int, where), vdim=_require(m, "vdim", int, where),
+            q_rank=_require(m, "q_rank", int, where), kv_rank=_require(m, "kv_rank", int, where),
+            scale=_require(m, "scale", float, where), rot_base=base, rot_dims=dims, rot_scaling=scaling)
+        if min(s.heads, s.dim, s.rot_dim, s.vdim, s.q_rank, s.kv_rank) <= 0:
+            raise ConfigError(f"{where}: heads, dim, rot_dim, vdim, q_rank and kv_rank must be > 0")
+        if s.rot_dims > s.rot_dim:
+            raise ConfigError(f"{where}: rot.dims {s.rot_dims} exceeds rot_dim {s.rot_dim}")
+        return s
+
+    def to_dict(self) -> Dict[str, Any]:
+        return {"heads": self.heads, "dim": self.dim, "rot_dim": self.rot_dim, "vdim": self.vdim, "q_rank": self.q_rank,
+                "kv_rank": self.kv_rank, "scale": self.scale, "rot": _llama3_rot_dict(self.rot_base, self.rot_dims, self.rot_scaling)}
+
+
+@dataclass(frozen=True)
+class SibodraFeedForwardSpec:
+    """``dense``: one gated feed-forward of width ``ff``.  ``moe``: ``experts`` feed-forwards without a gate of width ``ff``
+    each, of which a token uses ``top``, and a shared one of width ``shared_ff`` (0: none)."""
+    kind: str
+    ff: int
+    experts: int = 0
+    top: int = 0
+    shared_ff: int = 0
+
+    @staticmethod
+    def from_dict(mlp: Dict[str, Any], where: str) -> "SibodraFeedForwardSpec":
+        kind = _require(mlp, "kind", str, where)
+        if kind == "dense":
+            s = SibodraFeedForwardSpec("dense", _require(mlp, "ff", int, where))
+        elif kind == "moe":
+            router, shared = _obj(mlp, "router", where), mlp.get("shared")
+            if shared is not None and not isinstance(shared, dict):
+                raise ConfigError(f"{where}: 'shared' must be an object or null")
+            s = SibodraFeedForwardSpec(
+                "moe", _require(_obj(mlp, "expert", where), "ff", int, where + ".expert"),
+                _require(router, "experts", int, where + ".router"), _require(router, "top", int, where + ".router"),
+                _require(shared, "ff", int, where + ".shared") if shared is not None else 0)
+            if not (0 < s.top <= s.experts) or s.experts > 512:
+                raise ConfigError(f"{where}.router: need 0 < top <= experts <= 512")
+            if shared is not None and s.shared_ff <= 0:
+                raise ConfigError(f"{where}.shared: ff must be > 0")
+        else:
+            raise ConfigError(f"{where}: unknown feed-forward kind {kind!r} (known: dense, moe)")
+        if s.ff <= 0:
+            raise ConfigError(f"{where}: ff must be > 0")
+        return s
+
+    def to_dict(self) -> Dict[str, Any]:
+        if self.kind == "dense":
+            return {"kind": "dense", "ff": self.ff}
+        d = {"kind": "moe", "expert": {"ff": self.ff}, "router": {"experts": self.experts, "top": self.top}}
+        if self.shared_ff:
+            d["shared"] = {"ff": self.shared_ff}
+        return d
+
+
+SIBODRA_MIXERS = {"attention": CappedAttentionSpec, "latent_attention": QueryLatentAttentionSpec}
+MAX_STREAMS = 8
+
+
+@dataclass(frozen=True)
+class SibodraLayer:
+    mixer: Any                                        # one of the specs above
+    mlp: Optional[SibodraFeedForwardSpec] = None      # None: the layer has no feed-forward
+
+    @property
+    def type(self) -> str:
+        return self.mixer.kind
+
+
+@dataclass(frozen=True)
+class SibodraConfig(ModelConfig):
+    """``{"architecture": "Sibodra", "vocab", "width", "streams", "norm": {"eps"}, "logit_softcap",
+    "layers": [{"type", "mixer": {...}, "mlp": {...} | null}]}``.  The residual is ``streams`` rows a token that every
+    sub-layer reads and writes through small learned weights; the head has a matrix of its own and its logits are
+    soft-capped; no end-of-sequence token of its own."""
+
+    vocab_size: int = 0
+    hidden_size: int = 0
+    streams: int = 1
+    norm_eps: float = 1e-5
+    logit_softcap: Optional[float] = None
+    layers: tuple = ()
+    eos_token_ids: tuple = ()
+    architecture: str = "Sibodra"
+
+    @classmethod
+    def from_dict(cls, d: Dict[str, Any], where: str = "config.json") -> "SibodraConfig":
+        layers_in = d.get("layers")
+        if not isinstance(layers_in, list) or not layers_in:
+            raise ConfigError(f"{where}: 'layers' must be a non-empty list")
+        layers = []
+        for i, entry in enumerate(layers_in):
+            w = f"{where}.layers[{i}]"
+            if not isinstance(entry, dict):
+                raise ConfigError(f"{w}: must be an object")
+            kind = _require(entry, "type", str, w)
+            if kind not in SIBODRA_MIXERS:
+                raise ConfigError(f"{w}: unknown mixer type {kind!r} (known: {', '.join(sorted(SIBODRA_MIXERS))})")
+            mixer = SIBODRA_MIXERS[kind].from_dict(_obj(entry, "mixer", w), w + ".mixer")
+            mlp = entry.get("mlp")
+            if mlp is not None and not isinstance(mlp, dict):
+                raise ConfigError(f"{w}: 'mlp' must be null or an object")
+            layers.append(SibodraLayer(mixer, SibodraFeedForwardSpec.from_dict(mlp, w + ".mlp") if mlp is not None else None))
+        eos = d.get("eos_token_id")
+        eos_ids = () if eos is None else tuple(_typed(e, "eos_token_id", int, where) for e in (eos if isinstance(eos, list) else [eos]))
+        cap = d.get("logit_softcap")
+        cfg = cls(vocab_size=_require(d, "vocab", int, where), hidden_size=_require(d, "width", int, where),
+                  streams=_require(d, "streams", int, where), norm_eps=_require(_obj(d, "norm", where), "eps", float, where + ".norm"),
+                  logit_softcap=_typed(cap, "logit_softcap", float, where) if cap is not None else None,
+                  layers=tuple(layers), eos_token_ids=eos_ids)
+        if cfg.vocab_size <= 0 or cfg.hidden_size <= 0 or not cfg.norm_eps > 0:
+            raise ConfigError(f"{where}: vocab and width must be > 0, norm.eps > 0")
+        if not (1 <= cfg.streams <= MAX_STREAMS):
+            raise ConfigError(f"{where}: streams must be between 1 and {MAX_STREAMS}")
+        if cfg.logit_softcap is not None and not cfg.logit_softcap > 0:
+            raise ConfigError(f"{where}: logit_softcap must be > 0")
+        return cfg
+
+    def to_dict(self) -> Dict[str, Any]:
+        d: Dict[str, Any] = {
+            "architecture": self.architecture, "vocab": self.vocab_size, "width": self.hidden_size, "streams": self.streams,
+            "norm": {"eps": self.norm_eps},
+            "layers": [{"type": l.type, "mixer": l.mixer.to_dict(), "mlp": None if l.mlp is None else l.mlp.to_dict()}
+                       for l in self.layers]}
+        if self.logit_softcap is not None:
+            d["logit_softcap"] = self.logit_softcap
+        if self.eos_token_ids:
+            d["eos_token_id"] = list(self.eos_token_ids)
+        return d

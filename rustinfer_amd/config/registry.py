@@ -105,3 +105,4 @@ def _ensure_builtin() -> None:
     from ..models import pilavik  # noqa: F401  (registers Pilavik)
     from ..models import debuzen  # noqa: F401  (registers Debuzen)
     from ..models import zotonex  # noqa: F401  (registers Zotonex)
+    from ..models import sibodra  # noqa: F401  (registers Sibodra)

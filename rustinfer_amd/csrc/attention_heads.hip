@@ -3,17 +3,21 @@
 //
 //   head_norm_kv_write   queries and keys divided by their root mean square over the head, times a
 //                        weight of the head's size shared by all heads, the query times a
-//                        temperature that grows with the logarithm of its position; the query in
+//                        temperature that grows with the logarithm of its position, both turned by
+//                        their position over their first features; the query in
 //                        place, the normed key and the value into the token's page (a head may hold
 //                        several queries or keys side by side, each normed on its own);
 //   latent_kv_write      attention through one latent vector a token: the first R features of the
 //                        down projection are normed (c), the last r are one rotated key part for all
 //                        heads; the page takes the key [c, rotated part] and the value c; the
 //                        rotated part of every head's query goes to the tail of that head's
-//                        absorbed query [R + r];
+//                        absorbed query [R + r]; where the queries come from a latent of their own,
+//                        that latent is normed in the same pass (its product with the heads' matrix
+//                        comes after, and head_linear makes the tails);
 //   head_linear          out[t, h, :] = W_h x[t, h, :] for every head: the product that turns a
 //                        head's unrotated query into the latent space (W_uk,h^T q) and the weighted
-//                        sum of latents back into the head's value space (W_uv,h o).
+//                        sum of latents back into the head's value space (W_uv,h o), there times a
+//                        sigmoid a feature if the mixer has an output gate.
 //
 // Cache layout as everywhere: keys [pages][Hkv][page][dk], values [pages][Hkv][dv][page].
 #include "common.h"
@@ -30,7 +34,8 @@ __global__ __launch_bounds__(256) void head_norm_kv_write_kernel(
         T* __restrict__ q, int q_stride, const T* __restrict__ k, int k_stride, const T* __restrict__ v, int v_stride,
         int H, int Hkv, int dk, int dv, const float* __restrict__ qw, const float* __restrict__ kw, int do_norm, float eps,
         float temp_coef, int temp_every, const int* __restrict__ positions, const int* __restrict__ row_of_token,
-        T* __restrict__ kc, T* __restrict__ vc, const int* __restrict__ table, int max_blocks, int page, int write_kv, int maps) {
+        T* __restrict__ kc, T* __restrict__ vc, const int* __restrict__ table, int max_blocks, int page, int write_kv, int maps,
+        int rot, const float* __restrict__ cos_t, const float* __restrict__ sin_t) {
     const int t = blockIdx.x;
     const int b = row_of_token[t];
     if (b < 0) return;                       // padding token
@@ -55,7 +60,14 @@ __global__ __launch_bounds__(256) void head_norm_kv_write_kernel(
             ss = wave_sum(ss);
             f *= 1.f / sqrtf(ss / (float)dk + eps);
         }
-        for (int i = lane; i < dk; i += 64) {
+        const int half = rot >> 1;
+        for (int i = lane; i < half; i += 64) {            // a pair a lane: nobody else reads or writes its two features
+            const float a = ld_f32(src + i) * f * (w ? w[i] : 1.f), bb = ld_f32(src + i + half) * f * (w ? w[i + half] : 1.f);
+            const float c = cos_t[(size_t)pos * half + i], s = sin_t[(size_t)pos * half + i];
+            st_f32(dst + i, a * c - bb * s);
+            st_f32(dst + i + half, bb * c + a * s);
+        }
+        for (int i = rot + lane; i < dk; i += 64) {
             const float x = ld_f32(src + i);
             st_f32(dst + i, x * f * (w ? w[i] : 1.f));
         }
@@ -71,6 +83,7 @@ __global__ __launch_bounds__(256) void head_norm_kv_write_kernel(
 // ---------------------------------------------------------------------------
 // One block a token.  q [T][H (d + r)]: a head's unrotated features, then its r rotated ones, of which
 // the first `rot` are turned (feature i with i + rot/2).  down [T][R + r].  q_abs [T][H (R + r)].
+// q null: the heads' queries are not there yet.  ql [T][Rq] (or null): the queries' latent, normed into ql_out [T][Rq].
 // ---------------------------------------------------------------------------
 template <typename T>
 __global__ __launch_bounds__(256) void latent_kv_write_kernel(
@@ -78,7 +91,8 @@ __global__ __launch_bounds__(256) void latent_kv_write_kernel(
         int H, int d, int r, int R, int rot, const float* __restrict__ cw, float eps,
         const float* __restrict__ cos_t, const float* __restrict__ sin_t,
         const int* __restrict__ positions, const int* __restrict__ row_of_token,
-        T* __restrict__ kc, T* __restrict__ vc, const int* __restrict__ table, int max_blocks, int page, int write_kv) {
+        T* __restrict__ kc, T* __restrict__ vc, const int* __restrict__ table, int max_blocks, int page, int write_kv,
+        const T* __restrict__ ql, int ql_stride, int Rq, const float* __restrict__ qlw, T* __restrict__ ql_out, int qo_stride) {
     __shared__ float red[16];
     const int t = blockIdx.x;
     const int b = row_of_token[t];
@@ -93,11 +107,21 @@ __global__ __launch_bounds__(256) void latent_kv_write_kernel(
         if (rotate && j < rot) return ld_f32(part + j) * cs[j - half] + ld_f32(part + j - half) * sn[j - half];
         return ld_f32(part + j);
     };
-    const T* qrow = q + (size_t)t * q_stride;
-    T* qa = q_abs + (size_t)t * qa_stride;
-    for (int idx = threadIdx.x; idx < H * r; idx += 256) {
-        const int h = idx / r, j = idx - h * r;
-        st_f32(qa + h * (R + r) + R + j, turned(qrow + h * (d + r) + d, j));
+    if (q) {
+        const T* qrow = q + (size_t)t * q_stride;
+        T* qa = q_abs + (size_t)t * qa_stride;
+        for (int idx = threadIdx.x; idx < H * r; idx += 256) {
+            const int h = idx / r, j = idx - h * r;
+            st_f32(qa + h * (R + r) + R + j, turned(qrow + h * (d + r) + d, j));
+        }
+    }
+    if (ql) {
+        const T* row = ql + (size_t)t * ql_stride;
+        float ss = 0.f;
+        for (int i = threadIdx.x; i < Rq; i += 256) { const float x = ld_f32(row + i); ss = fmaf(x, x, ss); }
+        ss = block_sum(ss, red);
+        const float rs = 1.f / sqrtf(ss / (float)Rq + eps);
+        for (int i = threadIdx.x; i < Rq; i += 256) st_f32(ql_out + (size_t)t * qo_stride + i, ld_f32(row + i) * rs * (qlw ? qlw[i] : 1.f));
     }
     if (!write_kv) return;
     const int blk = table[(size_t)b * max_blocks + pos / page];
@@ -124,13 +148,43 @@ __global__ __launch_bounds__(256) void latent_kv_write_kernel(
 // ---------------------------------------------------------------------------
 constexpr int HL_T = 64, HL_N = 64, HL_K = 16;
 
+// What else a head's product may do.  tail > 0: the `tail` features behind the K that are multiplied go, turned by
+// the token's position (the first `rot` of them, feature i with i + rot/2), behind the N outputs.  gate (or null): output n of
+// head h is multiplied by sigmoid(gate[t * gate_stride + h * N + n]).
+template <typename T>
+struct HeadExtra {
+    int tail, rot, table_rows;
+    const float *cos_t, *sin_t;
+    const int* positions;
+    const T* gate;
+    int gate_stride;
+    __device__ __forceinline__ float gated(float v, int t, int at) const {
+        return gate ? v / (1.f + expf(-ld_f32(gate + (size_t)t * gate_stride + at))) : v;
+    }
+    // feature j of the tail that starts at `part`, for token t
+    __device__ __forceinline__ float turned(const T* part, int t, int j) const {
+        const int half = rot >> 1;
+        if (j >= 2 * half) return ld_f32(part + j);
+        const size_t at = (size_t)min(max(positions[t], 0), table_rows - 1) * half;
+        if (j < half) return ld_f32(part + j) * cos_t[at + j] - ld_f32(part + j + half) * sin_t[at + j];
+        return ld_f32(part + j) * cos_t[at + j - half] + ld_f32(part + j - half) * sin_t[at + j - half];
+    }
+};
+
 template <typename T>
 __global__ __launch_bounds__(256) void head_linear_kernel(
         const T* __restrict__ x, int x_stride, int x_head, const T* __restrict__ w, T* __restrict__ out, int out_stride,
-        int out_head, int Tn, int N, int K) {
+        int out_head, int Tn, int N, int K, HeadExtra<T> extra) {
     __shared__ float xs[HL_K][HL_T + 4];
     __shared__ float ws[HL_K][HL_N + 4];
     const int h = blockIdx.z, t0 = blockIdx.x * HL_T, n0 = blockIdx.y * HL_N;
+    if (n0 >= N) {                                     // the blocks of the tail (there are none without one)
+        for (int e = threadIdx.x; e < HL_T * extra.tail; e += 256) {
+            const int t = t0 + e / extra.tail, j = e % extra.tail;
+            if (t < Tn) st_f32(out + (size_t)t * out_stride + h * out_head + N + j, extra.turned(x + (size_t)t * x_stride + h * x_head + K, t, j));
+        }
+        return;
+    }
     const int tx = threadIdx.x & 15, ty = threadIdx.x >> 4;           // outputs 4 tx.., tokens 4 ty..
     const T* wh = w + (size_t)h * N * K;
     float acc[4][4] = {};
@@ -165,7 +219,7 @@ __global__ __launch_bounds__(256) void head_linear_kernel(
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
             const int n = n0 + 4 * tx + j;
-            if (n < N) st_f32(out + (size_t)t * out_stride + h * out_head + n, acc[i][j]);
+            if (n < N) st_f32(out + (size_t)t * out_stride + h * out_head + n, extra.gated(acc[i][j], t, h * N + n));
         }
     }
 }
@@ -191,8 +245,16 @@ __device__ __forceinline__ void hl_ld16(const bf16_t* p, float* f) {
 template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void head_linear_few_kernel(
         const T* __restrict__ x, int x_stride, int x_head, const T* __restrict__ w, T* __restrict__ out, int out_stride,
-        int out_head, int Tn, int N, int K) {
+        int out_head, int Tn, int N, int K, HeadExtra<T> extra) {
     constexpr int VL = VEC ? 16 / (int)sizeof(T) : 1;
+    if ((int)blockIdx.x * 32 >= N) {                   // the block of the tail (there is none without one)
+        const int h = blockIdx.y;
+        for (int e = threadIdx.x; e < Tn * extra.tail; e += 256) {
+            const int t = e / extra.tail, j = e % extra.tail;
+            st_f32(out + (size_t)t * out_stride + h * out_head + N + j, extra.turned(x + (size_t)t * x_stride + h * x_head + K, t, j));
+        }
+        return;
+    }
     const int h = blockIdx.y, part = threadIdx.x & 7, n = blockIdx.x * 32 + (threadIdx.x >> 3);
     const bool live = n < N;
     const T* wr = w + ((size_t)h * N + (live ? n : 0)) * K;
@@ -218,7 +280,7 @@ __global__ __launch_bounds__(256) void head_linear_few_kernel(
         float v = acc[t];
 #pragma unroll
         for (int o = 4; o > 0; o >>= 1) v += __shfl_xor(v, o, 8);
-        if (part == 0 && live) st_f32(out + (size_t)t * out_stride + h * out_head + n, v);
+        if (part == 0 && live) st_f32(out + (size_t)t * out_stride + h * out_head + n, extra.gated(v, t, h * N + n));
     }
 }
 
@@ -230,14 +292,18 @@ __global__ __launch_bounds__(256) void head_linear_few_kernel(
 // temp_every > 0: the query at position p is multiplied by 1 + temp_coef ln(floor((p + 1) / temp_every) + 1).
 // maps: queries a query head and keys a key head hold, side by side (q [T][>= H maps dk], k [T][>= Hkv maps dk]);
 // each is normed on its own with the same weight, and the cached key row has maps dk features.
+// rot > 0: behind the norm the first rot features of every query and key are turned by the token's position (feature i
+// with i + rot/2; tables [table_rows][rot / 2]).
 extern "C" int ri_head_norm_kv_write(
         void* q, int q_stride, const void* k, int k_stride, const void* v, int v_stride, int dtype, int T,
         int H, int Hkv, int dk, int dv, const float* qw, const float* kw, int do_norm, float eps,
         float temp_coef, int temp_every, const int* positions, const int* row_of_token,
-        void* kc, void* vc, int num_pages, const int* table, int max_blocks, int page, int write_kv, int maps, hipStream_t stream) {
+        void* kc, void* vc, int num_pages, const int* table, int max_blocks, int page, int write_kv, int maps,
+        int rot, const float* cos_t, const float* sin_t, int table_rows, hipStream_t stream) {
     RI_REQUIRE(T >= 0 && H > 0 && Hkv > 0 && dk > 0 && dv > 0 && page > 0 && maps > 0, "ri_head_norm_kv_write: bad sizes");
     RI_REQUIRE(q_stride >= H * maps * dk, "ri_head_norm_kv_write: query row stride %d too small", q_stride);
     RI_REQUIRE(!do_norm || eps > 0.f, "ri_head_norm_kv_write: eps must be > 0");
+    RI_REQUIRE(rot == 0 || (rot > 0 && rot % 2 == 0 && rot <= dk && cos_t && sin_t && table_rows > 0), "ri_head_norm_kv_write: rot %d must be even and within the key size %d, with tables", rot, dk);
     if (write_kv) RI_REQUIRE(k && v && kc && vc && table && max_blocks > 0 && num_pages > 0 && k_stride >= Hkv * maps * dk && v_stride >= Hkv * dv,
                              "ri_head_norm_kv_write: no keys, values or cache given, or their row strides too small");
     if (T == 0) return 0;
@@ -246,32 +312,35 @@ extern "C" int ri_head_norm_kv_write(
     const int by = T <= 256 ? min(((H + Hkv) * maps + 3) / 4, 64) : 1;
     const dim3 grid(T, by);
     if (dtype == RI_F32)
-        head_norm_kv_write_kernel<float><<<grid, 256, 0, stream>>>((float*)q, q_stride, (const float*)k, k_stride, (const float*)v, v_stride, H, Hkv, dk, dv, qw, kw, do_norm, eps, temp_coef, temp_every, positions, row_of_token, (float*)kc, (float*)vc, table, max_blocks, page, write_kv, maps);
+        head_norm_kv_write_kernel<float><<<grid, 256, 0, stream>>>((float*)q, q_stride, (const float*)k, k_stride, (const float*)v, v_stride, H, Hkv, dk, dv, qw, kw, do_norm, eps, temp_coef, temp_every, positions, row_of_token, (float*)kc, (float*)vc, table, max_blocks, page, write_kv, maps, rot, cos_t, sin_t);
     else if (dtype == RI_BF16)
-        head_norm_kv_write_kernel<bf16_t><<<grid, 256, 0, stream>>>((bf16_t*)q, q_stride, (const bf16_t*)k, k_stride, (const bf16_t*)v, v_stride, H, Hkv, dk, dv, qw, kw, do_norm, eps, temp_coef, temp_every, positions, row_of_token, (bf16_t*)kc, (bf16_t*)vc, table, max_blocks, page, write_kv, maps);
+        head_norm_kv_write_kernel<bf16_t><<<grid, 256, 0, stream>>>((bf16_t*)q, q_stride, (const bf16_t*)k, k_stride, (const bf16_t*)v, v_stride, H, Hkv, dk, dv, qw, kw, do_norm, eps, temp_coef, temp_every, positions, row_of_token, (bf16_t*)kc, (bf16_t*)vc, table, max_blocks, page, write_kv, maps, rot, cos_t, sin_t);
     else
         return ri_fail("ri_head_norm_kv_write: unknown dtype %d", dtype);
     RI_LAUNCHED("ri_head_norm_kv_write");
     return 0;
 }
 
-// The cache belongs to one key/value head with keys of R + r features and values of R.
+// The cache belongs to one key/value head with keys of R + r features and values of R.  q null: no queries' tails.
+// ql [T][>= Rq] (null: none): rows that are divided by their root mean square and multiplied by qlw into ql_out.
 extern "C" int ri_latent_kv_write(
         const void* q, int q_stride, const void* down, int down_stride, void* q_abs, int qa_stride, int dtype, int T,
         int H, int d, int r, int R, int rot, const float* cw, float eps, const float* cos_t, const float* sin_t, int table_rows,
         const int* positions, const int* row_of_token, void* kc, void* vc, int num_pages,
-        const int* table, int max_blocks, int page, int write_kv, hipStream_t stream) {
+        const int* table, int max_blocks, int page, int write_kv,
+        const void* ql, int ql_stride, int Rq, const float* qlw, void* ql_out, int qo_stride, hipStream_t stream) {
     RI_REQUIRE(T >= 0 && H > 0 && d >= 0 && r >= 0 && R > 0 && page > 0, "ri_latent_kv_write: bad sizes");
-    RI_REQUIRE(q_stride >= H * (d + r) && qa_stride >= H * (R + r) && down_stride >= R + r, "ri_latent_kv_write: row strides too small");
+    RI_REQUIRE((!q || (q_stride >= H * (d + r) && qa_stride >= H * (R + r))) && down_stride >= R + r, "ri_latent_kv_write: row strides too small");
     RI_REQUIRE(eps > 0.f, "ri_latent_kv_write: eps must be > 0");
     if (cos_t) RI_REQUIRE(rot > 0 && rot % 2 == 0 && rot <= r && sin_t && table_rows > 0, "ri_latent_kv_write: rot %d must be even and within the rotated part %d", rot, r);
     if (write_kv) RI_REQUIRE(kc && vc && table && max_blocks > 0 && num_pages > 0, "ri_latent_kv_write: no cache given");
     if (T == 0) return 0;
-    RI_REQUIRE(q && down && q_abs && positions && row_of_token, "ri_latent_kv_write: null pointer");
+    RI_REQUIRE((!q || q_abs) && down && positions && row_of_token, "ri_latent_kv_write: null pointer");
+    RI_REQUIRE(!ql || (ql_out && Rq > 0 && ql_stride >= Rq && qo_stride >= Rq), "ri_latent_kv_write: the queries' latent needs a place and row strides of at least its size");
     if (dtype == RI_F32)
-        latent_kv_write_kernel<float><<<T, 256, 0, stream>>>((const float*)q, q_stride, (const float*)down, down_stride, (float*)q_abs, qa_stride, H, d, r, R, rot, cw, eps, cos_t, sin_t, positions, row_of_token, (float*)kc, (float*)vc, table, max_blocks, page, write_kv);
+        latent_kv_write_kernel<float><<<T, 256, 0, stream>>>((const float*)q, q_stride, (const float*)down, down_stride, (float*)q_abs, qa_stride, H, d, r, R, rot, cw, eps, cos_t, sin_t, positions, row_of_token, (float*)kc, (float*)vc, table, max_blocks, page, write_kv, (const float*)ql, ql_stride, Rq, qlw, (float*)ql_out, qo_stride);
     else if (dtype == RI_BF16)
-        latent_kv_write_kernel<bf16_t><<<T, 256, 0, stream>>>((const bf16_t*)q, q_stride, (const bf16_t*)down, down_stride, (bf16_t*)q_abs, qa_stride, H, d, r, R, rot, cw, eps, cos_t, sin_t, positions, row_of_token, (bf16_t*)kc, (bf16_t*)vc, table, max_blocks, page, write_kv);
+        latent_kv_write_kernel<bf16_t><<<T, 256, 0, stream>>>((const bf16_t*)q, q_stride, (const bf16_t*)down, down_stride, (bf16_t*)q_abs, qa_stride, H, d, r, R, rot, cw, eps, cos_t, sin_t, positions, row_of_token, (bf16_t*)kc, (bf16_t*)vc, table, max_blocks, page, write_kv, (const bf16_t*)ql, ql_stride, Rq, qlw, (bf16_t*)ql_out, qo_stride);
     else
         return ri_fail("ri_latent_kv_write: unknown dtype %d", dtype);
     RI_LAUNCHED("ri_latent_kv_write");
@@ -279,20 +348,24 @@ extern "C" int ri_latent_kv_write(
 }
 
 // x [T][x_stride], head h at column h * x_head; w [H][N][K] contiguous; out [T][out_stride], head h
-// at column h * out_head.
+// at column h * out_head.  tail, rot, the tables and the gate: see HeadExtra.
 extern "C" int ri_head_linear(const void* x, int x_stride, int x_head, const void* w, void* out, int out_stride, int out_head,
-                              int dtype, int T, int H, int N, int K, hipStream_t stream) {
+                              int dtype, int T, int H, int N, int K, int tail, int rot, const float* cos_t, const float* sin_t, int table_rows,
+                              const int* positions, const void* gate, int gate_stride, hipStream_t stream) {
     RI_REQUIRE(T >= 0 && H > 0 && N > 0 && K > 0, "ri_head_linear: bad sizes T=%d H=%d N=%d K=%d", T, H, N, K);
-    RI_REQUIRE(x_head >= 0 && out_head >= 0 && x_stride >= (H - 1) * x_head + K && out_stride >= (H - 1) * out_head + N,
+    RI_REQUIRE(tail >= 0 && rot >= 0 && rot % 2 == 0 && rot <= tail && (rot == 0 || (cos_t && sin_t && table_rows > 0 && positions)), "ri_head_linear: a tail of %d with %d turned features", tail, rot);
+    RI_REQUIRE(!gate || gate_stride >= H * N, "ri_head_linear: the gate's row stride is too small");
+    RI_REQUIRE(x_head >= 0 && out_head >= 0 && x_stride >= (H - 1) * x_head + K + tail && out_stride >= (H - 1) * out_head + N + tail,
                "ri_head_linear: row strides too small");
     if (T == 0) return 0;
     RI_REQUIRE(x && w && out, "ri_head_linear: null pointer");
     RI_REQUIRE(H <= 65535 && (N + HL_N - 1) / HL_N <= 65535, "ri_head_linear: too many heads or outputs for the grid");
     if (T <= HLF_T) {
-        const dim3 few((N + 31) / 32, H);
+        const dim3 few((N + 31) / 32 + (tail > 0), H);
         const int vl = dtype == RI_F32 ? 4 : 8;
         const bool vec = K % vl == 0 && x_stride % vl == 0 && x_head % vl == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)w % 16 == 0;
-#define RI_HLF(TT, VV) head_linear_few_kernel<TT, VV><<<few, 256, 0, stream>>>((const TT*)x, x_stride, x_head, (const TT*)w, (TT*)out, out_stride, out_head, T, N, K)
+#define RI_HLF(TT, VV) head_linear_few_kernel<TT, VV><<<few, 256, 0, stream>>>((const TT*)x, x_stride, x_head, (const TT*)w, (TT*)out, out_stride, out_head, T, N, K, \
+                                      HeadExtra<TT>{tail, rot, table_rows, cos_t, sin_t, positions, (const TT*)gate, gate_stride})
         if (dtype == RI_F32) { if (vec) RI_HLF(float, true); else RI_HLF(float, false); }
         else if (dtype == RI_BF16) { if (vec) RI_HLF(bf16_t, true); else RI_HLF(bf16_t, false); }
         else
@@ -301,11 +374,13 @@ extern "C" int ri_head_linear(const void* x, int x_stride, int x_head, const voi
         RI_LAUNCHED("ri_head_linear");
         return 0;
     }
-    const dim3 grid((T + HL_T - 1) / HL_T, (N + HL_N - 1) / HL_N, H);
+    const dim3 grid((T + HL_T - 1) / HL_T, (N + HL_N - 1) / HL_N + (tail > 0), H);
     if (dtype == RI_F32)
-        head_linear_kernel<float><<<grid, 256, 0, stream>>>((const float*)x, x_stride, x_head, (const float*)w, (float*)out, out_stride, out_head, T, N, K);
+        head_linear_kernel<float><<<grid, 256, 0, stream>>>((const float*)x, x_stride, x_head, (const float*)w, (float*)out, out_stride, out_head, T, N, K,
+            HeadExtra<float>{tail, rot, table_rows, cos_t, sin_t, positions, (const float*)gate, gate_stride});
     else if (dtype == RI_BF16)
-        head_linear_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)x, x_stride, x_head, (const bf16_t*)w, (bf16_t*)out, out_stride, out_head, T, N, K);
+        head_linear_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)x, x_stride, x_head, (const bf16_t*)w, (bf16_t*)out, out_stride, out_head, T, N, K,
+            HeadExtra<bf16_t>{tail, rot, table_rows, cos_t, sin_t, positions, (const bf16_t*)gate, gate_stride});
     else
         return ri_fail("ri_head_linear: unknown dtype %d", dtype);
     RI_LAUNCHED("ri_head_linear");

@@ -1,5 +1,5 @@
-// What the attention kernels over the paged cache share: which keys a query sees, and how the outputs of
-// a head's two softmax maps become one.
+// What the attention kernels over the paged cache share: which keys a query sees, what happens to scores and
+// outputs, and how the outputs of a head's two softmax maps become one.
 #pragma once
 #include "common.h"
 
@@ -9,6 +9,17 @@ __device__ __forceinline__ int aw_first_key(int p, int window, int chunk) {
     if (chunk > 0) lo = max(lo, p - p % chunk);
     return lo;
 }
+
+// What a head's output is multiplied by after the softmax: the sigmoid of one logit a token and head (token t, head h at
+// gate[t * stride + h]); no gate: 1.
+template <typename T>
+struct HeadGate {
+    const T* gate;
+    int stride;
+    __device__ __forceinline__ float at(int t, int head) const {
+        return gate ? 1.f / (1.f + expf(-ld_f32(gate + (size_t)t * stride + head))) : 1.f;
+    }
+};
 
 // How the outputs of a head's two maps become one (maps = 2).
 struct DiffHow { float lam, gain, eps; };

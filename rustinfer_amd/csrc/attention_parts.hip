@@ -8,7 +8,8 @@
 //
 // Keys in sight, heads of two maps and their difference: attention_masks.h, attention_window.hip (which
 // takes what these kernels do not: 32-bit storage, turned values, kept first positions, sigmoid
-// weights, other page sizes).  A sink joins the denominator at the end.
+// weights, other page sizes).  A sink joins the denominator at the end.  Scores may be soft-capped, c tanh(s / c), and
+// a head's output may be multiplied by a sigmoid (HeadGate).
 // Cache layout: keys [pages][Hkv][page][maps dk], values [pages][Hkv][dv][page]; pages of a multiple of 16.
 //
 // Nothing but the final outputs passes through LDS.  The accumulator of S^T = K Q^T holds one query a
@@ -54,6 +55,16 @@ __device__ __forceinline__ bf16x8_t zero8() {
     return __builtin_bit_cast(bf16x8_t, ri_u32x4_t{0u, 0u, 0u, 0u});
 }
 
+// Scores from the products of queries and keys, in the log2 domain: scale, or the soft cap c tanh(s / c) as
+// c (1 - 2 / (1 + exp(2 s / c))).
+struct ScoreHow {
+    float scale_log2e;      // what a product is multiplied by (1 behind a cap, which leaves log2 units)
+    float cap_log2e, cap_k; // c log2(e) (0: no cap), and 2 scale log2(e) / c
+    __device__ __forceinline__ float cap(float s) const {
+        return cap_log2e * fmaf(-2.f, __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(s * cap_k)), 1.f);
+    }
+};
+
 // 1 / denominator of a map from its reference m (log2 domain) and sum l, a sink (natural domain) joining
 __device__ __forceinline__ float ap_final(float m, float l, const float* __restrict__ sink, int vh) {
     if (!(l > 0.f)) return 0.f;
@@ -74,8 +85,9 @@ __global__ __launch_bounds__(256, FT <= 4 && DU <= 8 ? 2 : 1) void attn_parts_pr
         const bf16_t* __restrict__ q, int q_stride, bf16_t* __restrict__ out, int out_stride,
         const bf16_t* __restrict__ kc, const bf16_t* __restrict__ vc, const int* __restrict__ table, int max_blocks,
         const int* __restrict__ cu_q, const int* __restrict__ q_start, const int* __restrict__ kv_lens,
-        int num_rows, int H, int Hkv, int dk, int dv, int page, float scale_log2e, int window, int chunk, int maps, DiffHow diff,
-        const float* __restrict__ sink, int tiles) {
+        int num_rows, int H, int Hkv, int dk, int dv, int page, ScoreHow how, int window, int chunk, int maps, DiffHow diff,
+        const float* __restrict__ sink, HeadGate<bf16_t> hgate, int tiles) {
+    const float scale_log2e = how.scale_log2e;
     extern __shared__ __align__(16) float lds[];       // [4 waves][32][dv + 4]: the outputs, after the last keys
     const int G = H / Hkv, HB = G < 4 ? G : 4, SB = 4 / HB, TQB = 32 * SB;
     // Blocks of one key/value head are Hkv apart (with eight heads: an XCD's L2 each).  A late tile sees many keys, an
@@ -168,6 +180,10 @@ __global__ __launch_bounds__(256, FT <= 4 && DU <= 8 ? 2 : 1) void attn_parts_pr
             pages_of(key0 + 32, na, nb);
             load_keys(key0 + 32, na, nb, kf);
         }
+        if (how.cap_log2e > 0.f) {
+#pragma unroll
+            for (int i = 0; i < 16; ++i) s[i] = how.cap(s[i]);
+        }
         // register i: key key0 + 16 (i / 8) + 8 lh + i % 8, for the lane's query
         if (key0 < hot_lo || key0 >= hot_hi) {
 #pragma unroll
@@ -224,7 +240,8 @@ __global__ __launch_bounds__(256, FT <= 4 && DU <= 8 ? 2 : 1) void attn_parts_pr
         pb = nb;
     }
     l += __shfl_xor(l, 32, 64);
-    const float inv = ap_final(m, l, sink, vh);
+    float inv = ap_final(m, l, sink, vh);
+    if (lq < ntw) inv *= hgate.at(t0w + lq, vh);           // (one map a head)
     const int os = dv + 4;
     float* ow = lds + (size_t)wave * 32 * os;
     if (wave_on) {
@@ -274,7 +291,7 @@ template <int KU, int VU>
 __global__ __launch_bounds__(64) void attn_parts_decode_kernel(
         const bf16_t* __restrict__ q, int q_stride, const bf16_t* __restrict__ kc, const bf16_t* __restrict__ vc,
         const int* __restrict__ table, int max_blocks, const int* __restrict__ cu_q, const int* __restrict__ q_start,
-        const int* __restrict__ kv_lens, int H, int Hkv, int dk, int dv, int page, float scale_log2e, int window, int chunk, int maps,
+        const int* __restrict__ kv_lens, int H, int Hkv, int dk, int dv, int page, ScoreHow how, int window, int chunk, int maps,
         int slots, int CG, float* __restrict__ part_ml, float* __restrict__ part_o) {
     const int G = H / Hkv, b = blockIdx.z, g = blockIdx.y / CG, c0 = (blockIdx.y % CG) * 16;
     const int lane = threadIdx.x, col = lane & 15, grp = lane >> 4;
@@ -340,7 +357,7 @@ __global__ __launch_bounds__(64) void attn_parts_decode_kernel(
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const int key = c_lo + 32 * (tl >> 1) + 8 * grp + 4 * (tl & 1) + i;
-                s[tl][i] = key >= j0 && key < visible ? s[tl][i] * scale_log2e : -INFINITY;
+                s[tl][i] = key >= j0 && key < visible ? (how.cap_log2e > 0.f ? how.cap(s[tl][i]) : s[tl][i] * how.scale_log2e) : -INFINITY;
                 m_new = fmaxf(m_new, s[tl][i]);
             }
         m_new = fmaxf(m_new, __shfl_xor(m_new, 16, 64));
@@ -407,7 +424,8 @@ template <int NC, int MAPS>
 __global__ __launch_bounds__(256) void attn_parts_combine_kernel(
         const float* __restrict__ part_ml, const float* __restrict__ part_o, bf16_t* __restrict__ out, int out_stride,
         const int* __restrict__ cu_q, const int* __restrict__ q_start, const int* __restrict__ kv_lens,
-        int H, int dv, int window, int chunk, int slots, DiffHow diff, const float* __restrict__ sink) {
+        int H, int dv, int window, int chunk, int slots, DiffHow diff, const float* __restrict__ sink,
+        HeadGate<bf16_t> hgate) {
     __shared__ float wts[MAPS][AP_SLOTS];
     __shared__ float acc_s[4][MAPS][64 * NC];
     const int b = blockIdx.y, ho = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -422,6 +440,7 @@ __global__ __launch_bounds__(256) void attn_parts_combine_kernel(
         const float m = lane < n ? part_ml[(at + lane) * 2] : -INFINITY, l = lane < n ? part_ml[(at + lane) * 2 + 1] : 0.f;
         const float M = wave_max(m), w = lane < n ? __builtin_amdgcn_exp2f(m - M) : 0.f;
         fin[k] = ap_final(M, wave_sum(w * l), sink, ho * MAPS + k);
+        if (MAPS == 1) fin[k] *= hgate.at(t, ho);
         if (wave == 0 && lane < AP_SLOTS) wts[k][lane] = w;
     }
     __syncthreads();
@@ -483,15 +502,19 @@ extern "C" size_t ri_attention_parts_workspace(int T, int H, int dv, int maps, i
 
 // bfloat16 attention of the step's tokens over the cache; arguments as ri_attention_window's.
 // single_tokens != 0: every row has at most one token, row b's is token cu_q[b] (workspace needed).
+// softcap > 0: a score s becomes softcap tanh(s / softcap).  gate [T][>= H] (null: none) with a row stride: a head's
+// output is multiplied by the sigmoid of its number there (maps = 1).
 extern "C" int ri_attention_parts(
         const void* q, int q_stride, void* out, int out_stride, const void* kc, const void* vc, int num_pages, int page,
         int H, int Hkv, int dk, int dv, const int* table, int max_blocks, const int* cu_q, const int* q_start, const int* kv_lens,
         int num_rows, int T, float scale, int window, int chunk, int maps, float diff_lam, float diff_gain, float diff_eps,
-        const float* sink, int single_tokens, int max_kv_len, float* workspace, size_t workspace_floats, hipStream_t stream) {
+        const float* sink, float softcap, const void* gate, int gate_stride, int single_tokens, int max_kv_len, float* workspace,
+        size_t workspace_floats, hipStream_t stream) {
     RI_REQUIRE(ri_attention_parts_supported(H, Hkv, dk, dv, maps, page), "ri_attention_parts: sizes not taken (H=%d Hkv=%d dk=%d dv=%d maps=%d page=%d)", H, Hkv, dk, dv, maps, page);
     RI_REQUIRE(T >= 0 && num_rows >= 0 && max_blocks > 0 && num_pages > 0 && window >= 0 && chunk >= 0, "ri_attention_parts: bad sizes");
     RI_REQUIRE(maps == 1 || diff_eps > 0.f, "ri_attention_parts: the difference of two maps takes an eps > 0");
     RI_REQUIRE(q_stride >= H * maps * dk && out_stride >= H * dv && q_stride % 8 == 0, "ri_attention_parts: row strides too small, or a query stride that is no multiple of 8");
+    RI_REQUIRE(softcap >= 0.f && (!gate || (maps == 1 && gate_stride >= H)), "ri_attention_parts: softcap must be >= 0; a gate goes with one map a head and a row stride of at least the heads");
     if (T == 0 || num_rows == 0) return 0;
     RI_REQUIRE(q && out && kc && vc && table && cu_q && q_start && kv_lens, "ri_attention_parts: null pointer");
     RI_REQUIRE((uintptr_t)q % 16 == 0 && (uintptr_t)kc % 16 == 0 && (uintptr_t)vc % 16 == 0, "ri_attention_parts: operands must be aligned to 16 bytes");
@@ -501,7 +524,8 @@ extern "C" int ri_attention_parts(
     const bf16_t* kb = (const bf16_t*)kc;
     const bf16_t* vb = (const bf16_t*)vc;
     bf16_t* ob = (bf16_t*)out;
-    const float sl = scale * LOG2E;
+    const ScoreHow how{softcap > 0.f ? 1.f : scale * LOG2E, softcap * LOG2E, softcap > 0.f ? 2.f * scale * LOG2E / softcap : 0.f};
+    const HeadGate<bf16_t> hgate{(const bf16_t*)gate, gate_stride};
     if (single_tokens) {
         const int slots = ap_slots(window, chunk, max_kv_len), CG = (G + 15) / 16;
         RI_REQUIRE(workspace && max_kv_len > 0 && workspace_floats >= (size_t)T * Hm * slots * (dv + 2), "ri_attention_parts: workspace of %zu floats for %d slots", workspace_floats, slots);
@@ -512,14 +536,14 @@ extern "C" int ri_attention_parts(
         auto part = KU <= 2 ? (VU <= 4 ? attn_parts_decode_kernel<2, 4> : VU <= 8 ? attn_parts_decode_kernel<2, 8> : attn_parts_decode_kernel<2, 16>)
                   : KU <= 4 ? (VU <= 4 ? attn_parts_decode_kernel<4, 4> : VU <= 8 ? attn_parts_decode_kernel<4, 8> : attn_parts_decode_kernel<4, 16>)
                             : (VU <= 4 ? attn_parts_decode_kernel<8, 4> : VU <= 8 ? attn_parts_decode_kernel<8, 8> : attn_parts_decode_kernel<8, 16>);
-        part<<<dim3(slots, Hkv * CG, num_rows), 64, 0, stream>>>(qb, q_stride, kb, vb, table, max_blocks, cu_q, q_start, kv_lens, Hm, Hkv, dk, dv, page, sl,
+        part<<<dim3(slots, Hkv * CG, num_rows), 64, 0, stream>>>(qb, q_stride, kb, vb, table, max_blocks, cu_q, q_start, kv_lens, Hm, Hkv, dk, dv, page, how,
                                                                  window, chunk, maps, slots, CG, part_ml, part_o);
         const int NC = (dv + 63) / 64;
 #define RI_AP_COMBINE(MM) (NC == 1 ? attn_parts_combine_kernel<1, MM> : NC == 2 ? attn_parts_combine_kernel<2, MM> \
                          : NC == 3 ? attn_parts_combine_kernel<3, MM> : attn_parts_combine_kernel<4, MM>)
         auto combine = maps == 2 ? RI_AP_COMBINE(2) : RI_AP_COMBINE(1);
 #undef RI_AP_COMBINE
-        combine<<<dim3(H, num_rows), 256, 0, stream>>>(part_ml, part_o, ob, out_stride, cu_q, q_start, kv_lens, Hm, dv, window, chunk, slots, diff, sink);
+        combine<<<dim3(H, num_rows), 256, 0, stream>>>(part_ml, part_o, ob, out_stride, cu_q, q_start, kv_lens, Hm, dv, window, chunk, slots, diff, sink, hgate);
         RI_LAUNCHED("ri_attention_parts");
         return 0;
     }
@@ -537,7 +561,7 @@ extern "C" int ri_attention_parts(
             } \
         } \
         kernel<<<dim3(tiles * Hkv, (G + 3) / 4), 256, lds, stream>>>(qb, q_stride, ob, out_stride, kb, vb, table, max_blocks, cu_q, q_start, kv_lens, num_rows, \
-            Hm, Hkv, dk, dv, page, sl, window, chunk, maps, diff, sink, tiles); } while (0)
+            Hm, Hkv, dk, dv, page, how, window, chunk, maps, diff, sink, hgate, tiles); } while (0)
 #define RI_AP_F(D) do { if (FT <= 2) RI_AP(D, 2); else if (FT <= 4) RI_AP(D, 4); else RI_AP(D, 8); } while (0)
     if (DU <= 4) RI_AP_F(4);
     else if (DU <= 8) RI_AP_F(8);

@@ -15,6 +15,8 @@
 // of a head is a head of its own (2 H of them) whose keys are its map's half of the key row.  A head's output is
 // the difference of its two maps' outputs, o = a - lam b, divided by its root mean square over the
 // head's dv values (diff_eps inside the root) and multiplied by diff_gain; a and b stay 32-bit.
+// cap > 0: a score s becomes cap tanh(s / cap) before anything else looks at it.  A head's output may be
+// multiplied by a sigmoid (HeadGate; one map a head, no turned values).
 // Storage is 32-bit or bfloat16; scores, weights, sums and the turns are 32-bit.
 // Cache layout: keys [pages][Hkv][page][dk], values [pages][Hkv][dv][page] (positions of a
 // feature contiguous).
@@ -127,10 +129,15 @@ __global__ __launch_bounds__(256) void rotate_kv_write_kernel(
     }
 }
 
+__device__ __forceinline__ float aw_score(float dot, float scale, float cap) {
+    const float s = dot * scale;
+    return cap > 0.f ? cap * tanhf(s / cap) : s;
+}
+
 // One row's scores against the keys of a block, one key a lane: the block's maximum, the weights
 // relative to it and their sum.  m_b = -inf (l_b = 0) if the row sees no key of the block.
-__device__ __forceinline__ float aw_block_scores(float dot, bool mine, float scale, float& m_b, float& l_b) {
-    const float sc = mine ? dot * scale : -INFINITY;
+__device__ __forceinline__ float aw_block_scores(float dot, bool mine, float scale, float cap, float& m_b, float& l_b) {
+    const float sc = mine ? aw_score(dot, scale, cap) : -INFINITY;
     m_b = wave_max(sc);
     float pj = 0.f;
     if (m_b > -INFINITY) pj = mine ? expf(sc - m_b) : 0.f;
@@ -141,8 +148,8 @@ __device__ __forceinline__ float aw_block_scores(float dot, bool mine, float sca
 // The same for weights that are sigmoids of the scores plus a number a head, with no normalisation over
 // the keys: the block's "maximum" is 0 where the row sees a key of it, so that merging adds the blocks' sums
 // as they are (exp(0 - 0) = 1), and the result is the sum itself (aw_final_factor gives 1).
-__device__ __forceinline__ float aw_block_sigmoids(float dot, bool mine, float scale, float bias, float& m_b, float& l_b) {
-    const float pj = mine ? 1.f / (1.f + expf(-(dot * scale + bias))) : 0.f;
+__device__ __forceinline__ float aw_block_sigmoids(float dot, bool mine, float scale, float cap, float bias, float& m_b, float& l_b) {
+    const float pj = mine ? 1.f / (1.f + expf(-(aw_score(dot, scale, cap) + bias))) : 0.f;
     m_b = __any(mine) ? 0.f : -INFINITY;
     l_b = wave_sum(pj);
     return pj;
@@ -190,7 +197,7 @@ __global__ __launch_bounds__(256) void attn_window_kernel(
         const int* __restrict__ cu_q, const int* __restrict__ q_start, const int* __restrict__ kv_lens,
         int num_rows, int H, int Hkv, int dk, int dv, int page, float scale, int window, int TQ, int NK,
         const float* __restrict__ vcos, const float* __restrict__ vsin, int v_interleaved, const float* __restrict__ sink,
-        int keep, const float* __restrict__ sig_bias, int chunk, int maps, DiffHow diff) {
+        int keep, const float* __restrict__ sig_bias, int chunk, int maps, DiffHow diff, float cap, HeadGate<T> hgate) {
     extern __shared__ __align__(16) float lds[];
     // (maps = 2: map m of a key lies at m * dkp of its row)
     const int dkp = (dk + 3) & ~3, dkr = maps * dk, ks_stride = maps * dkp + 4, vs_stride = dv + 1;
@@ -333,8 +340,8 @@ __global__ __launch_bounds__(256) void attn_window_kernel(
             for (int rb = 0; rb < 4; ++rb) {
                 const int i = 4 * bi + rb;
                 const bool mine = lane < NK && (j >= row_lo[i] || j < keep) && j < row_hi[i];
-                const float pj = sig_bias ? aw_block_sigmoids(s[rb], mine, scale, sig_bias[g * G + (wave + 4 * i) % G], m_b[i], l_b[i])
-                                          : aw_block_scores(s[rb], mine, scale, m_b[i], l_b[i]);
+                const float pj = sig_bias ? aw_block_sigmoids(s[rb], mine, scale, cap, sig_bias[g * G + (wave + 4 * i) % G], m_b[i], l_b[i])
+                                          : aw_block_scores(s[rb], mine, scale, cap, m_b[i], l_b[i]);
                 if (lane < NK) Ps[(wave + 4 * i) * NK + lane] = pj;
             }
         }
@@ -403,10 +410,11 @@ __global__ __launch_bounds__(256) void attn_window_kernel(
             if (r >= R) continue;
             T* o = out + (size_t)(t0 + r / G) * out_stride + (g * G + r % G) * dv;
             const float fin = sig_bias ? 1.f : sink ? aw_final_factor(m[i], l[i], sink, g * G + r % G) : 0.f;
+            const float gate = hgate.at(t0 + r / G, g * G + r % G);
 #pragma unroll
             for (int c = 0; c < NC; ++c) {
                 const int d = lane + 64 * c;
-                if (d < dv) st_f32(o + d, (sink || sig_bias) ? acc[i][c] * fin : (l[i] > 0.f ? acc[i][c] / l[i] : 0.f));
+                if (d < dv) st_f32(o + d, ((sink || sig_bias) ? acc[i][c] * fin : (l[i] > 0.f ? acc[i][c] / l[i] : 0.f)) * gate);
             }
         }
         return;
@@ -455,7 +463,7 @@ __global__ __launch_bounds__(64) void attn_window_combine_kernel(
         const int* __restrict__ cu_q, const int* __restrict__ q_start, const int* __restrict__ kv_lens,
         int H, int dv, int window, int NK, int slots,
         const float* __restrict__ vcos, const float* __restrict__ vsin, int v_interleaved, const float* __restrict__ sink,
-        int keep, int sigmoid_weights, int chunk, DiffHow diff) {
+        int keep, int sigmoid_weights, int chunk, DiffHow diff, HeadGate<T> hgate) {
     __shared__ float Os[256];
     const int b = blockIdx.y, ho = blockIdx.x, lane = threadIdx.x;
     const int t = cu_q[b];
@@ -511,11 +519,12 @@ __global__ __launch_bounds__(64) void attn_window_combine_kernel(
         aw_write_difference<T, NC>(o, acc[0], acc[1], dv, lane, diff);
         return;
     }
+    const float gate = hgate.at(t, ho);
 #pragma unroll
     for (int c = 0; c < NC; ++c) {
         const int d = lane + 64 * c;
         if (d < dv) {
-            const float y = sigmoid_weights ? acc[0][c] : sink ? acc[0][c] * aw_final_factor(m[0], l[0], sink, ho) : (l[0] > 0.f ? acc[0][c] / l[0] : 0.f);
+            const float y = (sigmoid_weights ? acc[0][c] : sink ? acc[0][c] * aw_final_factor(m[0], l[0], sink, ho) : (l[0] > 0.f ? acc[0][c] / l[0] : 0.f)) * gate;
             if (vcos == nullptr) st_f32(o + d, y);
             else Os[d] = y;
         }
@@ -546,7 +555,7 @@ __global__ __launch_bounds__(256) void attn_window_decode_kernel(
         const int* __restrict__ table, int max_blocks, const int* __restrict__ cu_q, const int* __restrict__ q_start,
         const int* __restrict__ kv_lens, int H, int Hkv, int dk, int dv, int page, float scale, int window, int slots,
         float* __restrict__ part_ml, float* __restrict__ part_o, int heads_a_wave, int keep, const float* __restrict__ sig_bias,
-        int chunk) {
+        int chunk, float cap) {
     extern __shared__ __align__(16) float lds[];       // [4 waves][G][64] weights
     // many query heads a key/value head (one shared latent, say): the heads are dealt to several
     // blocks in stretches of heads_a_wave, each reading the block of keys for its own heads
@@ -614,8 +623,8 @@ __global__ __launch_bounds__(256) void attn_window_decode_kernel(
         for (int rb = 0; rb < 4; ++rb) {
             if (h0 + rb >= h_hi) break;
             float m_b, l_b;
-            Ps[(h0 + rb) * AD_KEYS + lane] = sig_bias ? aw_block_sigmoids(s[rb], mine, scale, sig_bias[g * G + h0 + rb], m_b, l_b)
-                                                      : aw_block_scores(s[rb], mine, scale, m_b, l_b);
+            Ps[(h0 + rb) * AD_KEYS + lane] = sig_bias ? aw_block_sigmoids(s[rb], mine, scale, cap, sig_bias[g * G + h0 + rb], m_b, l_b)
+                                                      : aw_block_scores(s[rb], mine, scale, cap, m_b, l_b);
             if (lane == 0) {
                 float* dst = part_ml + (at0 + (size_t)(h0 + rb) * slots) * 2;
                 dst[0] = m_b;
@@ -767,7 +776,7 @@ int aw_launch(const T* q, int q_stride, T* out, int out_stride, const T* kc, con
               const int* cu_q, const int* q_start, const int* kv_lens, int num_rows, int Tn, int H, int Hkv, int dk, int dv,
               int page, float scale, int window, const float* vcos, const float* vsin, int v_interleaved,
               int slots, float* workspace, const float* sink, int keep, const float* sig_bias,
-              int chunk, int maps, DiffHow diff, hipStream_t stream) {
+              int chunk, int maps, DiffHow diff, float cap, HeadGate<T> hgate, hipStream_t stream) {
     const int G = H / Hkv, TQ = AW_ROWS / G;           // (H: the maps of all heads)
     const int NK = aw_keys_a_block(dk, dv, maps);
     const size_t lds = aw_lds_bytes(dk, dv, NK, maps);
@@ -801,17 +810,17 @@ int aw_launch(const T* q, int q_stride, T* out, int out_stride, const T* kc, con
         RI_REQUIRE((long)Hkv * stretches <= 65535, "ri_attention_window: too many heads for the grid");
         part<<<dim3((slots + 3) / 4, Hkv * stretches, num_rows), 256, sizeof(float) * 4 * G * AD_KEYS, stream>>>(
             q, q_stride, kc, vc, table, max_blocks, cu_q, q_start, kv_lens, H, Hkv, dk, dv, page, scale, window, slots, part_ml, part_o,
-            heads_a_wave, keep, sig_bias, chunk);
+            heads_a_wave, keep, sig_bias, chunk, cap);
         auto combine = RI_AW_FORM(attn_window_combine_kernel);
 #undef RI_AW_FORM
         combine<<<dim3(H / maps, num_rows), 64, 0, stream>>>(part_ml, part_o, out, out_stride, cu_q, q_start, kv_lens, H, dv, window, AD_KEYS, slots,
-                                                             vcos, vsin, v_interleaved, sink, keep, sig_bias != nullptr, chunk, diff);
+                                                             vcos, vsin, v_interleaved, sink, keep, sig_bias != nullptr, chunk, diff, hgate);
         return 0;
     }
     const int tiles = (Tn + TQ - 1) / TQ + num_rows;   // at most: every request may end in a short tile
     kernel<<<dim3(tiles, Hkv), 256, lds, stream>>>(q, q_stride, out, out_stride, kc, vc, table, max_blocks, cu_q, q_start, kv_lens,
                                                    num_rows, H, Hkv, dk, dv, page, scale, window, TQ, NK, vcos, vsin, v_interleaved, sink,
-                                                   keep, sig_bias, chunk, maps, diff);
+                                                   keep, sig_bias, chunk, maps, diff, cap, hgate);
     return 0;
 }
 }  // namespace
@@ -835,16 +844,20 @@ extern "C" size_t ri_attention_window_workspace(int T, int H, int dv, int window
 // chunk: a query sees keys of its own chunk of so many positions only (0: no chunks).
 // maps = 2: q [T][>= H 2 dk], keys of 2 dk features, sinks and biases [2 H]; a head's output is
 // gain (a - lam b) / rms(a - lam b) with a, b its two maps' outputs (diff_eps inside the root; no turned values then).
+// softcap > 0: a score s becomes softcap tanh(s / softcap).  gate [T][>= H] of the activations' dtype (null: none): a head's
+// output is multiplied by the sigmoid of its number there (maps = 1, no turned values).
 extern "C" int ri_attention_window(
         const void* q, int q_stride, void* out, int out_stride, int dtype, const void* kc, const void* vc,
         int num_pages, int page, int H, int Hkv, int dk, int dv, const int* table, int max_blocks,
         const int* cu_q, const int* q_start, const int* kv_lens, int num_rows, int T,
         float scale, int window, const float* vcos, const float* vsin, int v_table_rows, int v_interleaved,
         int single_tokens, int max_kv_len, float* workspace, size_t workspace_floats, const float* sink,
-        int keep, const float* sig_bias, int chunk, int maps, float diff_lam, float diff_gain, float diff_eps, hipStream_t stream) {
+        int keep, const float* sig_bias, int chunk, int maps, float diff_lam, float diff_gain, float diff_eps,
+        float softcap, const void* gate, int gate_stride, hipStream_t stream) {
     RI_REQUIRE(ri_attention_window_supported(H, Hkv, dk, dv, maps), "ri_attention_window: sizes not taken (H=%d Hkv=%d dk=%d dv=%d maps=%d)", H, Hkv, dk, dv, maps);
     RI_REQUIRE(keep >= 0 && chunk >= 0 && !(sink && sig_bias), "ri_attention_window: keep and chunk must be >= 0, and sigmoid weights take no sink");
     RI_REQUIRE(maps == 1 || (!vcos && diff_eps > 0.f), "ri_attention_window: the difference of two maps takes no turned values and an eps > 0");
+    RI_REQUIRE(softcap >= 0.f && (!gate || (maps == 1 && !vcos && gate_stride >= H)), "ri_attention_window: softcap must be >= 0; a gate goes with one map a head, no turned values and a row stride of at least the heads");
     if (window == 0 && chunk == 0) keep = 0;
     RI_REQUIRE(T >= 0 && num_rows >= 0 && max_blocks > 0 && num_pages > 0 && window >= 0 && page > 0, "ri_attention_window: bad sizes");
     RI_REQUIRE(q_stride >= H * maps * dk && out_stride >= H * dv, "ri_attention_window: row strides too small");
@@ -862,9 +875,9 @@ extern "C" int ri_attention_window(
     const DiffHow diff{diff_lam, diff_gain, diff_eps};
     int rc;
     if (dtype == RI_F32)
-        rc = aw_launch<float>((const float*)q, q_stride, (float*)out, out_stride, (const float*)kc, (const float*)vc, table, max_blocks, cu_q, q_start, kv_lens, num_rows, T, H * maps, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, slots, workspace, sink, keep, sig_bias, chunk, maps, diff, stream);
+        rc = aw_launch<float>((const float*)q, q_stride, (float*)out, out_stride, (const float*)kc, (const float*)vc, table, max_blocks, cu_q, q_start, kv_lens, num_rows, T, H * maps, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, slots, workspace, sink, keep, sig_bias, chunk, maps, diff, softcap, HeadGate<float>{(const float*)gate, gate_stride}, stream);
     else if (dtype == RI_BF16)
-        rc = aw_launch<bf16_t>((const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)kc, (const bf16_t*)vc, table, max_blocks, cu_q, q_start, kv_lens, num_rows, T, H * maps, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, slots, workspace, sink, keep, sig_bias, chunk, maps, diff, stream);
+        rc = aw_launch<bf16_t>((const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)kc, (const bf16_t*)vc, table, max_blocks, cu_q, q_start, kv_lens, num_rows, T, H * maps, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, slots, workspace, sink, keep, sig_bias, chunk, maps, diff, softcap, HeadGate<bf16_t>{(const bf16_t*)gate, gate_stride}, stream);
     else
         return ri_fail("ri_attention_window: unknown dtype %d", dtype);
     if (rc) return rc;
@@ -906,7 +919,7 @@ __global__ __launch_bounds__(256) void attn_window_mfma_kernel(
         const int* __restrict__ cu_q, const int* __restrict__ q_start, const int* __restrict__ kv_lens,
         int num_rows, int H, int Hkv, int dk, int dv, int page, float scale, int window,
         const float* __restrict__ vcos, const float* __restrict__ vsin, int v_interleaved, const float* __restrict__ sink,
-        int keep, const float* __restrict__ sig_bias, int chunk, int maps, DiffHow diff) {
+        int keep, const float* __restrict__ sig_bias, int chunk, int maps, DiffHow diff, float cap, HeadGate<T> hgate) {
     extern __shared__ __align__(16) float lds[];
     constexpr int DKP = 8 * QU;
     const int KS = maps * DKP + 4, dkr = maps * dk;    // (maps = 2: map m of a key lies at m * DKP of its row)
@@ -1042,6 +1055,10 @@ __global__ __launch_bounds__(256) void attn_window_mfma_kernel(
                 s = __builtin_amdgcn_mfma_f32_32x32x2f32(k4.z, qr[u * 4 + 2], s, 0, 0, 0);
                 s = __builtin_amdgcn_mfma_f32_32x32x2f32(k4.w, qr[u * 4 + 3], s, 0, 0, 0);
             }
+            if (cap > 0.f) {
+#pragma unroll
+                for (int i = 0; i < 16; ++i) s[i] = cap * tanhf(s[i] / cap);
+            }
             // register i: key kt0 + 8 (i / 4) + 4 lh + i % 4, for the lane's query
             const int j_lo = q_first, j_hi = min(pq + 1, kv_len);
             float mt = -INFINITY;
@@ -1090,7 +1107,8 @@ __global__ __launch_bounds__(256) void attn_window_mfma_kernel(
     }
     // the sums of a query lie in the lane of its lower and of its upper half: add the two l
     l += __shfl_xor(l, 32, 64);
-    const float inv = sig_bias ? 1.f : aw_final_factor(m, l, sink, head);
+    float inv = sig_bias ? 1.f : aw_final_factor(m, l, sink, head);
+    if (row_on) inv *= hgate.at(t0w + lq, head);       // (one map a head)
     __syncthreads();                                   // the last keys and values have been used
     float* ow = Os + (size_t)wave * 32 * dv;
     if (wave_on) {
@@ -1142,7 +1160,7 @@ template <typename T, int QU, int FT>
 int am_launch_as(const T* q, int q_stride, T* out, int out_stride, const T* kc, const T* vc, const int* table, int max_blocks,
                  const int* cu_q, const int* q_start, const int* kv_lens, int num_rows, int Tn, int H, int Hkv, int dk, int dv,
                  int page, float scale, int window, const float* vcos, const float* vsin, int v_interleaved, const float* sink,
-                 int keep, const float* sig_bias, int chunk, int maps, DiffHow diff, hipStream_t stream) {
+                 int keep, const float* sig_bias, int chunk, int maps, DiffHow diff, float cap, HeadGate<T> hgate, hipStream_t stream) {
     const int G = H / Hkv, HB = G < 4 ? G : 4, SB = 4 / HB, TQB = 32 * SB;      // (H: the maps of all heads)
     const size_t lds = am_lds_bytes(QU, dv, maps);
     auto kernel = attn_window_mfma_kernel<T, QU, FT>;
@@ -1156,7 +1174,7 @@ int am_launch_as(const T* q, int q_stride, T* out, int out_stride, const T* kc, 
     }
     const int tiles = (Tn + TQB - 1) / TQB + num_rows;
     kernel<<<dim3(tiles, Hkv, (G + 3) / 4), 256, lds, stream>>>(q, q_stride, out, out_stride, kc, vc, table, max_blocks, cu_q, q_start,
-                                                               kv_lens, num_rows, H, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, sink, keep, sig_bias, chunk, maps, diff);
+                                                               kv_lens, num_rows, H, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, sink, keep, sig_bias, chunk, maps, diff, cap, hgate);
     return 0;
 }
 
@@ -1164,9 +1182,9 @@ template <typename T>
 int am_launch(const T* q, int q_stride, T* out, int out_stride, const T* kc, const T* vc, const int* table, int max_blocks,
               const int* cu_q, const int* q_start, const int* kv_lens, int num_rows, int Tn, int H, int Hkv, int dk, int dv,
               int page, float scale, int window, const float* vcos, const float* vsin, int v_interleaved, const float* sink,
-              int keep, const float* sig_bias, int chunk, int maps, DiffHow diff, hipStream_t stream) {
+              int keep, const float* sig_bias, int chunk, int maps, DiffHow diff, float cap, HeadGate<T> hgate, hipStream_t stream) {
 #define RI_AM(QU, FT) return am_launch_as<T, QU, FT>(q, q_stride, out, out_stride, kc, vc, table, max_blocks, cu_q, q_start, kv_lens, \
-        num_rows, Tn, H, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, sink, keep, sig_bias, chunk, maps, diff, stream)
+        num_rows, Tn, H, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, sink, keep, sig_bias, chunk, maps, diff, cap, hgate, stream)
     if (dk <= 64) { if (dv <= 64) RI_AM(8, 2); if (dv <= 128) RI_AM(8, 4); RI_AM(8, 8); }
     if (dk <= 128) { if (dv <= 64) RI_AM(16, 2); if (dv <= 128) RI_AM(16, 4); RI_AM(16, 8); }
     if (dv <= 64) RI_AM(32, 2);
@@ -1191,10 +1209,11 @@ extern "C" int ri_attention_window_mfma(
         const int* cu_q, const int* q_start, const int* kv_lens, int num_rows, int T,
         float scale, int window, const float* vcos, const float* vsin, int v_table_rows, int v_interleaved,
         const float* sink, int keep, const float* sig_bias, int chunk, int maps, float diff_lam, float diff_gain, float diff_eps,
-        hipStream_t stream) {
+        float softcap, const void* gate, int gate_stride, hipStream_t stream) {
     RI_REQUIRE(ri_attention_window_mfma_supported(H, Hkv, dk, dv, maps), "ri_attention_window_mfma: sizes not taken (H=%d Hkv=%d dk=%d dv=%d maps=%d)", H, Hkv, dk, dv, maps);
     RI_REQUIRE(keep >= 0 && chunk >= 0 && !(sink && sig_bias), "ri_attention_window_mfma: keep and chunk must be >= 0, and sigmoid weights take no sink");
     RI_REQUIRE(maps == 1 || (!vcos && diff_eps > 0.f), "ri_attention_window_mfma: the difference of two maps takes no turned values and an eps > 0");
+    RI_REQUIRE(softcap >= 0.f && (!gate || (maps == 1 && !vcos && gate_stride >= H)), "ri_attention_window_mfma: softcap must be >= 0; a gate goes with one map a head, no turned values and a row stride of at least the heads");
     if (window == 0 && chunk == 0) keep = 0;
     RI_REQUIRE(T >= 0 && num_rows >= 0 && max_blocks > 0 && num_pages > 0 && window >= 0 && page > 0, "ri_attention_window_mfma: bad sizes");
     RI_REQUIRE(q_stride >= H * maps * dk && out_stride >= H * dv, "ri_attention_window_mfma: row strides too small");
@@ -1205,9 +1224,9 @@ extern "C" int ri_attention_window_mfma(
     const DiffHow diff{diff_lam, diff_gain, diff_eps};
     int rc;
     if (dtype == RI_F32)
-        rc = am_launch<float>((const float*)q, q_stride, (float*)out, out_stride, (const float*)kc, (const float*)vc, table, max_blocks, cu_q, q_start, kv_lens, num_rows, T, H * maps, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, sink, keep, sig_bias, chunk, maps, diff, stream);
+        rc = am_launch<float>((const float*)q, q_stride, (float*)out, out_stride, (const float*)kc, (const float*)vc, table, max_blocks, cu_q, q_start, kv_lens, num_rows, T, H * maps, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, sink, keep, sig_bias, chunk, maps, diff, softcap, HeadGate<float>{(const float*)gate, gate_stride}, stream);
     else if (dtype == RI_BF16)
-        rc = am_launch<bf16_t>((const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)kc, (const bf16_t*)vc, table, max_blocks, cu_q, q_start, kv_lens, num_rows, T, H * maps, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, sink, keep, sig_bias, chunk, maps, diff, stream);
+        rc = am_launch<bf16_t>((const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)kc, (const bf16_t*)vc, table, max_blocks, cu_q, q_start, kv_lens, num_rows, T, H * maps, Hkv, dk, dv, page, scale, window, vcos, vsin, v_interleaved, sink, keep, sig_bias, chunk, maps, diff, softcap, HeadGate<bf16_t>{(const bf16_t*)gate, gate_stride}, stream);
     else
         return ri_fail("ri_attention_window_mfma: unknown dtype %d", dtype);
     if (rc) return rc;

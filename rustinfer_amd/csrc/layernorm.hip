@@ -69,7 +69,9 @@ __global__ __launch_bounds__(BLOCK) void layer_norm_kernel(const float* __restri
     auto finish = [&](int i, const float* v) {
         float wv[VEC], bv[VEC], r[VEC];
         L::ld(w + i, wv);
-        L::ld(b + i, bv);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) bv[e] = 0.f;
+        if (b) L::ld(b + i, bv);
 #pragma unroll
         for (int e = 0; e < VEC; ++e) r[e] = (v[e] - mean) * rstd * wv[e] + bv[e];
         L::st(o + i, r);
@@ -274,7 +276,7 @@ extern "C" int ri_layer_norm(const float* x, const int* rows, const float* w, co
                              void* out, int out_dtype, int n_out, int d, hipStream_t stream) {
     RI_REQUIRE(n_out >= 0 && d > 0 && eps > 0.f, "ri_layer_norm: bad sizes rows=%d d=%d", n_out, d);
     if (n_out == 0) return 0;
-    RI_REQUIRE(x && w && b && out, "ri_layer_norm: null pointer");
+    RI_REQUIRE(x && w && out, "ri_layer_norm: null pointer");         // (b null: no bias)
     const bool v4 = d % 4 == 0 && aligned16(x) && aligned16(w) && aligned16(b) && vec4_ok(out, out_dtype);
     const bool wide = n_out <= FEW_ROWS && d >= 1024;
 #define RI_LN(TO, BLOCK, VEC) layer_norm_kernel<TO, BLOCK, VEC><<<n_out, BLOCK, 0, stream>>>(x, rows, w, b, eps, (TO*)out, d)

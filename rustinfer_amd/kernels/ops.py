@@ -1013,7 +1013,7 @@ def window_attention(q: torch.Tensor, out: torch.Tensor, H: int, Hkv: int, dk: i
                      ctx, scale: float, window: int = 0, value_rotary=None,
                      interleaved_values: bool = False, sink: Optional[torch.Tensor] = None,
                      keep_first: int = 0, sigmoid_bias: Optional[torch.Tensor] = None, chunk: int = 0,
-                     difference=None) -> None:
+                     difference=None, softcap: float = 0.0, gate: Optional[torch.Tensor] = None) -> None:
     """Attention of the step's tokens (rotated queries ``q [T, H dk]``) over the cache into
     ``out [T, H dv]``: keys of size ``dk``, values of size ``dv``, the last ``window`` positions
     (0: all).  ``value_rotary``: the cached values are turned by their positions, and each sum is
@@ -1025,8 +1025,15 @@ def window_attention(q: torch.Tensor, out: torch.Tensor, H: int, Hkv: int, dk: i
     positions only, counted from the request's first.  ``difference = (lam, gain, eps)``: every query head
     holds two queries and every key head two keys of ``dk`` features side by side (``q [T, H 2 dk]``, keys of
     ``2 dk``) over one value; with the two maps' outputs ``a``, ``b`` (32-bit) a head's output is
-    ``gain (a - lam b) / sqrt(mean((a - lam b)^2) + eps)``."""
-    _dev(q, out, k_cache, v_cache, block_table, sink, sigmoid_bias)
+    ``gain (a - lam b) / sqrt(mean((a - lam b)^2) + eps)``.  ``softcap`` (0: none): a score s becomes
+    ``softcap * tanh(s / softcap)``; a sink is not capped.  ``gate [T, H]`` (activations, columns of a wider buffer
+    allowed): each head's output is multiplied by the sigmoid of its number there."""
+    _dev(q, out, k_cache, v_cache, block_table, sink, sigmoid_bias, gate)
+    if gate is not None:
+        _rows2d(gate, "gate")
+        if difference is not None or value_rotary is not None or tuple(gate.shape) != (q.shape[0], H) or gate.dtype != q.dtype:
+            raise KernelError(f"window_attention: a gate is [T, {H}] of the queries' dtype, with one map a head and no turned values")
+    extras = (ctypes.c_float(softcap), _ptr(gate), gate.stride(0) if gate is not None else 0)
     maps = 2 if difference is not None else 1
     lam, gain, diff_eps = (ctypes.c_float(v) for v in (difference if difference is not None else (0.0, 1.0, 1.0)))
     if difference is not None and value_rotary is not None:
@@ -1063,7 +1070,7 @@ def window_attention(q: torch.Tensor, out: torch.Tensor, H: int, Hkv: int, dk: i
         _check(lib.ri_attention_parts(
             _ptr(q), q.stride(0), _ptr(out), out.stride(0), _ptr(k_cache), _ptr(v_cache), k_cache.shape[0], page,
             H, Hkv, dk, dv, _ptr(block_table), block_table.shape[1], _ptr(ctx.cu_q), _ptr(ctx.q_start), _ptr(ctx.kv_lens),
-            ctx.num_rows, T, ctypes.c_float(scale), int(window), int(chunk), maps, lam, gain, diff_eps, _ptr(sink),
+            ctx.num_rows, T, ctypes.c_float(scale), int(window), int(chunk), maps, lam, gain, diff_eps, _ptr(sink), *extras,
             single, int(ctx.max_kv_len), _ptr(ws), ctypes.c_size_t(need), _stream()))
         return
     if ctx.max_q_len > 1 and WINDOW_ATTENTION_MFMA and lib.ri_attention_window_mfma_supported(H, Hkv, dk, dv, maps):
@@ -1072,7 +1079,7 @@ def window_attention(q: torch.Tensor, out: torch.Tensor, H: int, Hkv: int, dk: i
             _ptr(q), q.stride(0), _ptr(out), out.stride(0), _dt(q), _ptr(k_cache), _ptr(v_cache), k_cache.shape[0], page,
             H, Hkv, dk, dv, _ptr(block_table), block_table.shape[1], _ptr(ctx.cu_q), _ptr(ctx.q_start), _ptr(ctx.kv_lens),
             ctx.num_rows, T, ctypes.c_float(scale), int(window), vcos, vsin, vrows, int(bool(interleaved_values)), _ptr(sink),
-            keep_first, _ptr(sigmoid_bias), int(chunk), maps, lam, gain, diff_eps, _stream()))
+            keep_first, _ptr(sigmoid_bias), int(chunk), maps, lam, gain, diff_eps, *extras, _stream()))
         return
     # a step of single tokens divides each row's keys between blocks, through a workspace
     ws, need = None, 0
@@ -1086,7 +1093,7 @@ def window_attention(q: torch.Tensor, out: torch.Tensor, H: int, Hkv: int, dk: i
         H, Hkv, dk, dv, _ptr(block_table), block_table.shape[1], _ptr(ctx.cu_q), _ptr(ctx.q_start), _ptr(ctx.kv_lens),
         ctx.num_rows, T, ctypes.c_float(scale), int(window), vcos, vsin, vrows, int(bool(interleaved_values)),
         single, int(ctx.max_kv_len), _ptr(ws), ctypes.c_size_t(need), _ptr(sink), keep_first, _ptr(sigmoid_bias),
-        int(chunk), maps, lam, gain, diff_eps, _stream()))
+        int(chunk), maps, lam, gain, diff_eps, *extras, _stream()))
 
 
 # ---------------------------------------------------------------------------
@@ -1176,13 +1183,14 @@ def head_norm_kv_write(q: torch.Tensor, k: Optional[torch.Tensor], v: Optional[t
                        dk: int, dv: int, q_weight: Optional[torch.Tensor], k_weight: Optional[torch.Tensor],
                        eps: float, positions: torch.Tensor, row_of_token: torch.Tensor, k_cache: torch.Tensor,
                        v_cache: torch.Tensor, block_table: torch.Tensor, page: int, write_kv: bool = True,
-                       norm: bool = True, temp_coef: float = 0.0, temp_every: int = 0, maps: int = 1) -> None:
+                       norm: bool = True, temp_coef: float = 0.0, temp_every: int = 0, maps: int = 1, rotary=None) -> None:
     """Every head of ``q [T, H dk]`` and ``k [T, Hkv dk]`` divided by its root mean square
     (``norm``), times a 32-bit weight of ``dk`` entries shared by the heads (or None); the query at
     position p also times ``1 + temp_coef ln(floor((p + 1) / temp_every) + 1)`` (``temp_every > 0``).
     q in place; k and ``v [T, Hkv dv]`` go into the token's page (``write_kv``).  ``maps``: a head holds so
     many queries or keys of ``dk`` features side by side (``q [T, H maps dk]``, ``k [T, Hkv maps dk]``), each
-    normed on its own."""
+    normed on its own.  ``rotary = (cos, sin, rot_dim)``: behind the norm the first ``rot_dim`` features of every
+    query and key are turned by the token's position (feature i with i + rot_dim/2)."""
     _dev(q, k, v, q_weight, k_weight, positions, row_of_token, k_cache, v_cache, block_table)
     _rows2d(q, "q")
     T = q.shape[0]
@@ -1201,32 +1209,51 @@ def head_norm_kv_write(q: torch.Tensor, k: Optional[torch.Tensor], v: Optional[t
         _i32(block_table, "block_table")
         if block_table.dim() != 2:
             raise KernelError("head_norm_kv_write: block_table must be [rows, max_blocks]")
+    rot, cos, sin, rows = 0, ctypes.c_void_p(0), ctypes.c_void_p(0), 0
+    if rotary is not None:
+        rot = int(rotary[2])
+        cos, sin, rows = _rot_tables(rotary, rot, "head_norm_kv_write")
     _check(_lib().ri_head_norm_kv_write(
         _ptr(q), q.stride(0), _ptr(k) if write_kv else ctypes.c_void_p(0), k.stride(0) if write_kv else 0,
         _ptr(v) if write_kv else ctypes.c_void_p(0), v.stride(0) if write_kv else 0, _dt(q), T, H, Hkv, dk, dv,
         _ptr(q_weight), _ptr(k_weight), int(bool(norm)), ctypes.c_float(eps), ctypes.c_float(temp_coef), int(temp_every),
         _ptr(positions), _ptr(row_of_token), _ptr(k_cache), _ptr(v_cache), k_cache.shape[0] if k_cache is not None else 0,
         _ptr(block_table), block_table.shape[1] if block_table is not None and block_table.dim() == 2 else 0, page,
-        int(bool(write_kv)), int(maps), _stream()))
+        int(bool(write_kv)), int(maps), rot, cos, sin, rows, _stream()))
 
 
-def latent_kv_write(q: torch.Tensor, down: torch.Tensor, q_abs: torch.Tensor, H: int, d: int, r: int, R: int,
+def latent_kv_write(q: Optional[torch.Tensor], down: torch.Tensor, q_abs: Optional[torch.Tensor], H: int, d: int, r: int, R: int,
                     latent_weight: Optional[torch.Tensor], eps: float, rotary, positions: torch.Tensor,
                     row_of_token: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
-                    block_table: torch.Tensor, page: int, write_kv: bool = True) -> None:
+                    block_table: torch.Tensor, page: int, write_kv: bool = True, query_latent=None) -> None:
     """Attention through a latent: ``down [T, R + r]`` holds the latent's R features, which are divided
     by their root mean square and multiplied by ``latent_weight`` (32-bit), and one rotated key part of
     r features; the page (one key/value head) takes the key ``[latent, turned part]`` and the value
     ``latent``.  ``q [T, H (d + r)]``: the turned rotated part of every head's query goes to the last r
     columns of that head in ``q_abs [T, H (R + r)]``.  ``rotary = (cos, sin, rot)`` turns the first
-    ``rot`` features of a rotated part (feature i with i + rot/2)."""
+    ``rot`` features of a rotated part (feature i with i + rot/2).
+    ``query_latent = (rows, weight, out)`` with ``q = q_abs = None``: the queries come from a latent of their own,
+    ``rows [T, Rq]``, which is normed the same way (32-bit ``weight`` of Rq entries) into ``out [T, Rq]``; the heads' queries
+    and their tails are made later (``head_linear``'s ``tail``)."""
     _dev(q, down, q_abs, latent_weight, positions, row_of_token, k_cache, v_cache, block_table)
-    for t, name in ((q, "q"), (down, "down"), (q_abs, "q_abs")):
-        _rows2d(t, name)
-    T = q.shape[0]
-    if q.shape[1] != H * (d + r) or tuple(down.shape) != (T, R + r) or tuple(q_abs.shape) != (T, H * (R + r)) \
-            or down.dtype != q.dtype or q_abs.dtype != q.dtype:
-        raise KernelError(f"latent_kv_write: q [T, {H * (d + r)}], down [T, {R + r}] and q_abs [T, {H * (R + r)}] of one dtype expected")
+    _rows2d(down, "down")
+    T, dt = down.shape[0], down.dtype
+    if down.shape[1] != R + r:
+        raise KernelError(f"latent_kv_write: down must be [T, {R + r}]")
+    if q is not None:
+        _rows2d(q, "q")
+        _rows2d(q_abs, "q_abs")
+        if tuple(q.shape) != (T, H * (d + r)) or tuple(q_abs.shape) != (T, H * (R + r)) or q.dtype != dt or q_abs.dtype != dt:
+            raise KernelError(f"latent_kv_write: q [T, {H * (d + r)}] and q_abs [T, {H * (R + r)}] of {dt} expected")
+    ql = qlw = ql_out = None
+    if query_latent is not None:
+        ql, qlw, ql_out = query_latent
+        _dev(ql, qlw, ql_out)
+        _rows2d(ql, "the queries' latent")
+        _rows2d(ql_out, "the queries' normed latent")
+        if ql.shape[0] != T or ql_out.shape != ql.shape or ql.dtype != dt or ql_out.dtype != dt:
+            raise KernelError(f"latent_kv_write: the queries' latent and its normed rows must be [T, n] of {dt}")
+        _f32_vec(qlw, ql.shape[1], "latent_kv_write: the queries' latent's weight")
     _i32(positions, "positions", T)
     _i32(row_of_token, "row_of_token", T)
     _f32_vec(latent_weight, R, "latent_kv_write: the latent's weight")
@@ -1235,62 +1262,85 @@ def latent_kv_write(q: torch.Tensor, down: torch.Tensor, q_abs: torch.Tensor, H:
         rot = int(rotary[2])
         cos, sin, rows = _rot_tables(rotary, rot, "latent_kv_write")
     if write_kv:
-        _check_cache_kv(k_cache, v_cache, 1, R + r, R, page, q.dtype, "latent_kv_write")
+        _check_cache_kv(k_cache, v_cache, 1, R + r, R, page, dt, "latent_kv_write")
         _i32(block_table, "block_table")
         if block_table.dim() != 2:
             raise KernelError("latent_kv_write: block_table must be [rows, max_blocks]")
     _check(_lib().ri_latent_kv_write(
-        _ptr(q), q.stride(0), _ptr(down), down.stride(0), _ptr(q_abs), q_abs.stride(0), _dt(q), T, H, d, r, R, rot,
+        _ptr(q), q.stride(0) if q is not None else 0, _ptr(down), down.stride(0), _ptr(q_abs), q_abs.stride(0) if q_abs is not None else 0,
+        _dt(down), T, H, d, r, R, rot,
         _ptr(latent_weight), ctypes.c_float(eps), cos, sin, rows, _ptr(positions), _ptr(row_of_token),
         _ptr(k_cache), _ptr(v_cache), k_cache.shape[0] if k_cache is not None else 0, _ptr(block_table),
-        block_table.shape[1] if block_table is not None and block_table.dim() == 2 else 0, page, int(bool(write_kv)), _stream()))
+        block_table.shape[1] if block_table is not None and block_table.dim() == 2 else 0, page, int(bool(write_kv)),
+        _ptr(ql), ql.stride(0) if ql is not None else 0, ql.shape[1] if ql is not None else 0, _ptr(qlw),
+        _ptr(ql_out), ql_out.stride(0) if ql_out is not None else 0, _stream()))
 
 
-def head_linear(x: torch.Tensor, x_head: int, w: torch.Tensor, out: torch.Tensor, out_head: int) -> None:
+def head_linear(x: torch.Tensor, x_head: int, w: torch.Tensor, out: torch.Tensor, out_head: int, tail: int = 0, rotary=None,
+                positions: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None) -> None:
     """``out[t, h * out_head : + N] = w[h] @ x[t, h * x_head : + K]`` for every head h; ``w [H, N, K]``.
-    x and out are 2-D with unit column stride (columns of wider buffers allowed); 32-bit sums."""
-    _dev(x, w, out)
+    x and out are 2-D with unit column stride (columns of wider buffers allowed); 32-bit sums.
+    ``tail`` > 0: the ``tail`` features behind the K of every head of x go behind the N of out, the first
+    ``rotary[2]`` of them turned by ``positions[t]`` (``rotary = (cos, sin, rot_dim)``, feature i with i + rot_dim/2).
+    ``gate [T, H N]``: every output is multiplied by the sigmoid of its number there."""
+    _dev(x, w, out, positions, gate)
     _rows2d(x, "x")
     _rows2d(out, "out")
     if w.dim() != 3 or not w.is_contiguous() or w.dtype != x.dtype or out.dtype != x.dtype or out.shape[0] != x.shape[0]:
         raise KernelError("head_linear: w must be contiguous [H, N, K] in the dtype of x and out")
     H, N, K = w.shape
-    if x.shape[1] < (H - 1) * x_head + K or out.shape[1] < (H - 1) * out_head + N:
+    if x.shape[1] < (H - 1) * x_head + K + tail or out.shape[1] < (H - 1) * out_head + N + tail:
         raise KernelError("head_linear: x or out is narrower than its heads")
+    rot, cos, sin, rows = 0, ctypes.c_void_p(0), ctypes.c_void_p(0), 0
+    if tail and rotary is not None:
+        rot = int(rotary[2])
+        cos, sin, rows = _rot_tables(rotary, rot, "head_linear")
+        _i32(positions, "positions", x.shape[0])
+    if gate is not None:
+        _rows2d(gate, "gate")
+        if tuple(gate.shape) != (x.shape[0], H * N) or gate.dtype != x.dtype:
+            raise KernelError(f"head_linear: the gate must be [T, {H * N}] of {x.dtype}")
     _check(_lib().ri_head_linear(_ptr(x), x.stride(0), int(x_head), _ptr(w), _ptr(out), out.stride(0), int(out_head),
-                                 _dt(x), x.shape[0], H, N, K, _stream()))
+                                 _dt(x), x.shape[0], H, N, K, int(tail), rot, cos, sin, rows, _ptr(positions) if rot else ctypes.c_void_p(0),
+                                 _ptr(gate), gate.stride(0) if gate is not None else 0, _stream()))
 
 
 # ---------------------------------------------------------------------------
 # a feed-forward of many experts
 # ---------------------------------------------------------------------------
+ROUTER_SCORES = {"softmax": 0, "sigmoid": 1, "chosen_softmax": 2}
+
+
 def _score_kind(score: str) -> int:
-    if score not in ("softmax", "sigmoid"):
-        raise KernelError(f"a router scores with 'softmax' or 'sigmoid', got {score!r}")
-    return int(score == "sigmoid")
+    if score not in ROUTER_SCORES:
+        raise KernelError(f"a router scores with one of {', '.join(ROUTER_SCORES)}, got {score!r}")
+    return ROUTER_SCORES[score]
 
 
-def _moe_widths(gate_up, act, E: int, F: int, shared: int, who: str):
+def _moe_widths(gate_up, act, E: int, F: int, shared: int, gated: bool, who: str):
     """The activations' width: the experts' ``E F`` columns, a shared expert's ``shared`` and zeros up to
     what ``act`` has."""
-    T, width = gate_up.shape[0], act.shape[1]
-    if gate_up.shape[1] != 2 * E * F + 2 * shared or act.shape[0] != T or width < E * F + shared or act.dtype != gate_up.dtype:
-        raise KernelError(f"{who}: gate_up [T, {2 * E * F + 2 * shared}] and act [T, >= {E * F + shared}] of one dtype expected")
+    T, width, cols = gate_up.shape[0], act.shape[1], (2 if gated else 1) * (E * F + shared)
+    if gate_up.shape[1] != cols or act.shape[0] != T or width < E * F + shared or act.dtype != gate_up.dtype:
+        raise KernelError(f"{who}: gate_up [T, {cols}] and act [T, >= {E * F + shared}] of one dtype expected")
     return T, width
 
 
 def moe_route(logits: torch.Tensor, weights: torch.Tensor, top: int, renormalize: bool = False,
-              score: str = "softmax", norm_eps: float = 0.0, scale: float = 1.0) -> None:
+              score: str = "softmax", norm_eps: float = 0.0, scale: float = 1.0, bias: Optional[torch.Tensor] = None) -> None:
     """``weights [T, E]`` (32-bit): ``softmax(logits)`` at the ``top`` largest entries of every row (ties:
     the lower index), 0 elsewhere; ``renormalize`` divides them by their sum (+ ``norm_eps``).
-    ``score = "sigmoid"``: the scores are ``sigmoid(logits)``, each on its own; ``scale`` multiplies the weights."""
-    _dev(logits, weights)
+    ``score = "sigmoid"``: the scores are ``sigmoid(logits)``, each on its own; ``scale`` multiplies the weights.
+    ``score = "chosen_softmax"``: the ``top`` largest logits are chosen and weighed by the softmax over them alone.
+    ``bias [E]`` (32-bit) is added to every row of logits first."""
+    _dev(logits, weights, bias)
+    _f32_vec(bias, logits.shape[1], "moe_route: the bias")
     _rows2d(logits, "logits")
     T, E = logits.shape
     if logits.dtype != torch.float32 or weights.dtype != torch.float32 or tuple(weights.shape) != (T, E) or not weights.is_contiguous():
         raise KernelError("moe_route: 32-bit logits [T, E] and contiguous 32-bit weights [T, E] expected")
     _check(_lib().ri_moe_route_as(_ptr(logits), logits.stride(0), _ptr(weights), T, E, int(top), int(bool(renormalize)),
-                                  _score_kind(score), ctypes.c_float(norm_eps), ctypes.c_float(scale), _stream()))
+                                  _score_kind(score), ctypes.c_float(norm_eps), ctypes.c_float(scale), _ptr(bias), _stream()))
 
 
 class ClippedGate:
@@ -1302,59 +1352,63 @@ class ClippedGate:
         self.shared_limit = float(limit if shared_limit is None else shared_limit)
 
 
-def _act_args(clip: Optional[ClippedGate], weigh_input: bool, shared_gate: Optional[torch.Tensor], T: int, who: str):
+def _act_args(clip: Optional[ClippedGate], weigh_input: bool, shared_gate: Optional[torch.Tensor], T: int, gated: bool, who: str):
     f = ctypes.c_float
     if shared_gate is not None and (shared_gate.dim() != 1 or shared_gate.shape[0] != T or shared_gate.dtype != torch.float32):
         raise KernelError(f"{who}: one 32-bit logit a token expected for the shared expert's gate")
-    how = (0, f(0), f(0), f(0), f(0)) if clip is None else (1, f(clip.limit), f(clip.shared_limit), f(clip.slope), f(clip.shift))
+    if not gated and clip is not None:
+        raise KernelError(f"{who}: the clipped activation belongs to experts with a gate")
+    how = (0 if gated else 2, f(0), f(0), f(0), f(0)) if clip is None else (1, f(clip.limit), f(clip.shared_limit), f(clip.slope), f(clip.shift))
     return how + (int(bool(weigh_input)), _ptr(shared_gate), shared_gate.stride(0) if shared_gate is not None else 0)
 
 
 def moe_swiglu_weighted(gate_up: torch.Tensor, weights: torch.Tensor, act: torch.Tensor, E: int, F: int,
                         shared: int = 0, clip: Optional[ClippedGate] = None, weigh_input: bool = False,
-                        shared_gate: Optional[torch.Tensor] = None) -> None:
+                        shared_gate: Optional[torch.Tensor] = None, gated: bool = True) -> None:
     """``act[t, e F + i] = weights[t, e] * silu(gate_up[t, e 2F + i]) * gate_up[t, e 2F + F + i]``.
     ``shared`` > 0: ``gate_up`` has ``2 shared`` more columns, a shared expert's gate and up, and ``act`` gets
     ``silu(gate) * up`` of them behind the experts' columns (weight 1, or the sigmoid of ``shared_gate [T]``, 32-bit
     logits of any stride); wider ``act``: zeros beyond.  ``clip``: the clipped activation instead of silu times
-    up.  ``weigh_input``: the weight multiplies an expert's gate and up values (its input) instead of the result."""
+    up.  ``weigh_input``: the weight multiplies an expert's gate and up values (its input) instead of the result.
+    ``gated = False``: experts (and a shared one) without a gate, ``relu(up)^2`` of ``gate_up [T, E F + shared]``."""
     _dev(gate_up, weights, act, shared_gate)
     _rows2d(gate_up, "gate_up")
     _rows2d(act, "act")
-    T, width = _moe_widths(gate_up, act, E, F, shared, "moe_swiglu_weighted")
+    T, width = _moe_widths(gate_up, act, E, F, shared, gated, "moe_swiglu_weighted")
     if weights.dtype != torch.float32 or tuple(weights.shape) != (T, E) or not weights.is_contiguous():
         raise KernelError("moe_swiglu_weighted: contiguous 32-bit weights [T, E] expected")
     _check(_lib().ri_moe_act_weighted(_ptr(gate_up), gate_up.stride(0), _ptr(weights), _ptr(act), act.stride(0),
                                       _dt(act), T, E, F, int(shared), width,
-                                      *_act_args(clip, weigh_input, shared_gate, T, "moe_swiglu_weighted"), _stream()))
+                                      *_act_args(clip, weigh_input, shared_gate, T, gated, "moe_swiglu_weighted"), _stream()))
 
 
 def moe_swiglu_routed(gate_up: torch.Tensor, logits: torch.Tensor, act: torch.Tensor, E: int, F: int, top: int,
                       renormalize: bool = False, score: str = "softmax", norm_eps: float = 0.0, scale: float = 1.0,
                       shared: int = 0, clip: Optional[ClippedGate] = None, weigh_input: bool = False,
-                      shared_gate: Optional[torch.Tensor] = None) -> None:
+                      shared_gate: Optional[torch.Tensor] = None, gated: bool = True, bias: Optional[torch.Tensor] = None) -> None:
     """``moe_route`` and ``moe_swiglu_weighted`` in one launch: the weights are made from the 32-bit
     ``logits [T, E]`` on the way and never stored."""
-    _dev(gate_up, logits, act, shared_gate)
+    _dev(gate_up, logits, act, shared_gate, bias)
+    _f32_vec(bias, E, "moe_swiglu_routed: the bias")
     _rows2d(gate_up, "gate_up")
     _rows2d(act, "act")
     _rows2d(logits, "logits")
-    T, width = _moe_widths(gate_up, act, E, F, shared, "moe_swiglu_routed")
+    T, width = _moe_widths(gate_up, act, E, F, shared, gated, "moe_swiglu_routed")
     if logits.dtype != torch.float32 or tuple(logits.shape) != (T, E):
         raise KernelError("moe_swiglu_routed: 32-bit logits [T, E] expected")
     _check(_lib().ri_moe_act_routed(_ptr(gate_up), gate_up.stride(0), _ptr(logits), logits.stride(0), _ptr(act),
                                     act.stride(0), _dt(act), T, E, F, int(top), int(bool(renormalize)),
-                                    _score_kind(score), ctypes.c_float(norm_eps), ctypes.c_float(scale),
+                                    _score_kind(score), ctypes.c_float(norm_eps), ctypes.c_float(scale), _ptr(bias),
                                     int(shared), width,
-                                    *_act_args(clip, weigh_input, shared_gate, T, "moe_swiglu_routed"), _stream()))
+                                    *_act_args(clip, weigh_input, shared_gate, T, gated, "moe_swiglu_routed"), _stream()))
 
 
 # ---------------------------------------------------------------------------
 # layer norm around gated sub-layers, a feed-forward that norms powers, a short convolution, the gated delta rule
 # ---------------------------------------------------------------------------
-def layer_norm(x: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor, eps: float, out: torch.Tensor,
+def layer_norm(x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor], eps: float, out: torch.Tensor,
                rows: Optional[torch.Tensor] = None) -> None:
-    """``out = (x - mean) / sqrt(var + eps) * weight + bias`` row by row; ``x`` 32-bit ``[T, d]``; with
+    """``out = (x - mean) / sqrt(var + eps) * weight + bias`` row by row (``bias = None``: none); ``x`` 32-bit ``[T, d]``; with
     ``rows`` (int32) only those rows, in that order."""
     _dev(x, weight, bias, out, rows)
     T, d = x.shape
@@ -1633,3 +1687,50 @@ def stream_pair(x: torch.Tensor, delta: Optional[torch.Tensor], y: torch.Tensor,
         ddt = _dt(delta)
     _check(_lib().ri_stream_pair(_ptr(x), _ptr(delta), ddt, parts, ctypes.c_longlong(stride), _ptr(y), F32, _ptr(out),
                                  _dt(out), T, d, _stream()))
+
+
+# ---------------------------------------------------------------------------
+# a residual stream of several rows a token
+# ---------------------------------------------------------------------------
+MAX_STREAMS = 8
+
+
+def hyper_streams(x: torch.Tensor, n: int, in_w: torch.Tensor, weight: torch.Tensor, eps: float, act: torch.Tensor,
+                  delta: Optional[torch.Tensor] = None, mix: Optional[torch.Tensor] = None, out_w: Optional[torch.Tensor] = None,
+                  bias: Optional[torch.Tensor] = None, streams_out: Optional[torch.Tensor] = None,
+                  rows: Optional[torch.Tensor] = None, centered: bool = True) -> None:
+    """What happens to the ``n`` residual rows of every token between two sub-layers, all in 32-bit:
+    ``new_t = sum_s mix[s, t] x_s + out_w[t] delta`` (without ``delta``: the streams as they are),
+    ``act = norm(sum_t in_w[t] new_t)``, the norm being a layer norm (``centered``; ``bias`` optional) or an RMS norm.
+    ``x``: ``[T, n, d]``, or ``[T, d]`` where all streams are still one row.  ``delta``: ``[T, d]`` or a 32-bit stack
+    ``[P, T, d]`` of partial sums.  ``streams_out [rows, n, d]`` (None: nobody reads them again) takes the new streams and
+    may be ``x``.  ``rows`` (int32): only those rows, in that order."""
+    _dev(x, in_w, weight, act, delta, mix, out_w, bias, streams_out, rows)
+    if x.dim() not in (2, 3) or x.dtype != torch.float32 or not x.is_contiguous() or (x.dim() == 3 and x.shape[1] != n):
+        raise KernelError(f"hyper_streams: contiguous 32-bit streams [T, {n}, d] or rows [T, d] expected")
+    T, d = x.shape[0], x.shape[-1]
+    n_out = rows.numel() if rows is not None else T
+    if rows is not None:
+        _i32(rows, "rows")
+    for v, size, name in ((in_w, n, "reading weights"), (out_w, n, "writing weights"), (mix, n * n, "mixing matrix"), (weight, d, "norm's weight"),
+                          (bias, d, "norm's bias")):
+        _f32_vec(v, size, f"hyper_streams: the {name}")
+    parts, stride, ddt = 1, 0, F32
+    if delta is not None:
+        if mix is None or out_w is None:
+            raise KernelError("hyper_streams: a delta needs its mixing matrix and writing weights")
+        if delta.dim() == 3:
+            parts, stride = delta.shape[0], delta.stride(0)
+        if delta.dim() not in (2, 3) or tuple(delta.shape[-2:]) != (T, d) or delta.stride(-1) != 1 or delta.stride(-2) != d \
+                or (delta.dim() == 3 and delta.dtype != torch.float32):
+            raise KernelError("hyper_streams: delta must be [T, d] or a float32 stack [P, T, d] with contiguous rows")
+        ddt = _dt(delta)
+    if tuple(act.shape) != (n_out, d) or not act.is_contiguous():
+        raise KernelError(f"hyper_streams: act must be contiguous [{n_out}, {d}]")
+    if streams_out is not None and (tuple(streams_out.shape) != (n_out, n, d) or streams_out.dtype != torch.float32 or not streams_out.is_contiguous()):
+        raise KernelError(f"hyper_streams: the new streams must be contiguous float32 [{n_out}, {n}, {d}]")
+    row, stream = (n * d, d) if x.dim() == 3 else (d, 0)
+    _check(_lib().ri_hyper_streams(
+        _ptr(x), ctypes.c_longlong(row), ctypes.c_longlong(stream), _ptr(rows), int(n), _ptr(delta), ddt, parts, ctypes.c_longlong(stride),
+        _ptr(mix), _ptr(out_w), _ptr(in_w), _ptr(streams_out), _ptr(weight), _ptr(bias), ctypes.c_float(eps), int(bool(centered)),
+        _ptr(act), _dt(act), n_out, d, _stream()))

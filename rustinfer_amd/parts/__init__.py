@@ -8,7 +8,8 @@ from .mlp import DenseMLP, MoEFeedForward, PolyNormMLP, SwiGLUMLP
 from .attention import LatentAttention, PagedAttention, WindowAttention
 from .recurrent import (ChannelGatedDeltaRule, GatedDeltaRule, GatedLinearAttention, GeneralDeltaRule, LightningAttention,
                         Retention, StateSpaceMixer)
-from .block import Hidden, ParallelBlock, PostNormBlock, PreNormBlock, SandwichBlock, TokenShift, TwoMixers
+from .block import (Hidden, HyperConnectedBlock, HyperConnection, ParallelBlock, PendingStreams, PostNormBlock, PreNormBlock,
+                    SandwichBlock, StreamsNorm, TokenShift, TwoMixers)
 from .registry import (MIXERS, FEED_FORWARDS, NORMS, POSITION_ENCODINGS, register_mixer,
                        register_feed_forward, register_norm, register_position_encoding,
                        make_part)

@@ -165,8 +165,8 @@ class WindowAttention(ProjectedPart, Mixer):
     ``qk_norm_eps``: queries and keys are divided by their root mean square over each head (this eps
     inside the root) and multiplied by weights of the head's size shared by all heads (tensors
     ``<q>.norm``, ``<k>.norm``); the cache holds the normed keys.  ``q_temperature = (coef, every)``:
-    the query at position p is multiplied by ``1 + coef ln(floor((p + 1) / every) + 1)``.  Either goes
-    without a rotation of queries and keys.  ``own_kv = False``: the layer has no keys and values of
+    the query at position p is multiplied by ``1 + coef ln(floor((p + 1) / every) + 1)``.  Both act before the
+    rotation, if there is one.  ``own_kv = False``: the layer has no keys and values of
     its own and reads a cache that another layer writes (the run order names it).
 
     ``interleaved``: the checkpoint's rotation pairs feature 2i with 2i + 1; the rows of ``q`` and ``k`` that make
@@ -174,7 +174,10 @@ class WindowAttention(ProjectedPart, Mixer):
     leaves every score as it was.  ``qk_unit_eps``: after the rotation every head of q and k is divided by its
     root mean square (this eps inside the root), with no weight.  ``keep_first``: behind the window the first so
     many positions of a sequence stay in sight, at their true positions; the cache never gives their pages back.
-    ``sink``: a learned number a head (tensor ``sink``) whose exponential joins the softmax's denominator.
+    ``sink``: a learned number a head (tensor ``sink``) whose exponential joins the softmax's denominator;
+    ``sink_score``: the same with one fixed number for all heads (0: the denominator has 1 added) and no tensor.
+    ``softcap``: a score s becomes ``softcap tanh(s / softcap)`` (a sink does not).  ``head_gate``: each head's output is
+    multiplied by the sigmoid of one more projection of the input (tensor ``g``, a row a head).
     ``sigmoid_weights``: no softmax; a visible key's weight is ``sigmoid(score + b_h)`` with a learned number a
     head (tensor ``pb``), and the weights are not normalised over the keys.
 
@@ -195,11 +198,19 @@ class WindowAttention(ProjectedPart, Mixer):
                  q_temperature=None, own_kv: bool = True, interleaved: bool = False,
                  qk_unit_eps: Optional[float] = None, keep_first: int = 0, sink: bool = False,
                  sigmoid_weights: bool = False, chunk: Optional[int] = None, difference: Optional[float] = None,
-                 difference_eps: float = 1e-5):
+                 difference_eps: float = 1e-5, sink_score: Optional[float] = None, softcap: Optional[float] = None,
+                 head_gate: bool = False):
         if num_heads % num_kv_heads:
             raise ValueError(f"num_heads {num_heads} is not a multiple of num_kv_heads {num_kv_heads}")
-        if sink and sigmoid_weights:
+        if (sink or sink_score is not None) and sigmoid_weights:
             raise ValueError("a sink belongs to a softmax: sigmoid weights take none")
+        if sink and sink_score is not None:
+            raise ValueError("a sink is learned or fixed, not both")
+        if head_gate and (difference is not None or value_pos_enc is not None):
+            raise ValueError("a gate a head goes with one map a head and without turned values")
+        self.sink_score = float(sink_score) if sink_score is not None else None
+        self.softcap = float(softcap) if softcap else 0.0
+        self.head_gate = bool(head_gate)
         if keep_first and not window and not chunk:
             keep_first = 0                       # without a window every position stays in sight anyway
         self.chunk = int(chunk) if chunk else None
@@ -216,8 +227,8 @@ class WindowAttention(ProjectedPart, Mixer):
         self.q_temperature = (float(q_temperature[0]), int(q_temperature[1])) if q_temperature else None
         self.own_kv = bool(own_kv)
         self.by_head = self.qk_norm_eps is not None or self.q_temperature is not None
-        if self.by_head and (pos_enc is not None or value_pos_enc is not None):
-            raise ValueError("a norm or a temperature on queries and keys goes without a rotation")
+        if self.by_head and value_pos_enc is not None:
+            raise ValueError("a norm or a temperature on queries and keys goes without turned values")
         self.hidden_size = int(hidden_size)
         self.num_heads, self.num_kv_heads = int(num_heads), int(num_kv_heads)
         self.head_dim, self.v_head_dim = int(head_dim), int(v_head_dim)
@@ -225,14 +236,14 @@ class WindowAttention(ProjectedPart, Mixer):
         self.window = int(window) if window else None
         self.pos_enc, self.value_pos_enc = pos_enc, value_pos_enc
         self.interleaved_values = bool(interleaved_values)
-        self.names = {"q": "q", "k": "k", "v": "v", "o": "o", "sink": "sink", "sigmoid_bias": "pb",
+        self.names = {"q": "q", "k": "k", "v": "v", "o": "o", "g": "g", "sink": "sink", "sigmoid_bias": "pb",
                       "lq1": "lq1", "lk1": "lk1", "lq2": "lq2", "lk2": "lk2"}
         if names:
             self.names.update(names)
         if self.maps == 2 and (pos_enc is not None or value_pos_enc is not None or not self.by_head):
             raise ValueError("the difference of two maps takes normed queries and keys without a rotation")
         if self.by_head and (self.interleaved or self.qk_unit_eps is not None):
-            raise ValueError("the weighted norm of queries and keys goes without a rotation and without the unit norm")
+            raise ValueError("the weighted norm of queries and keys goes without an interleaved rotation and without the unit norm")
 
     def arrange_in(self, name: str, w: torch.Tensor) -> torch.Tensor:
         rot = self.pos_enc.rot_dim if self.pos_enc is not None else 0
@@ -244,9 +255,10 @@ class WindowAttention(ProjectedPart, Mixer):
     def in_projections(self):
         n = self.names
         q, k = self.num_heads * self.maps * self.head_dim, self.num_kv_heads * self.maps * self.head_dim
+        gate = [(n["g"], self.num_heads)] if self.head_gate else []
         if not self.own_kv:
-            return [(n["q"], q)]
-        return [(n["q"], q), (n["k"], k), (n["v"], self.num_kv_heads * self.v_head_dim)]
+            return [(n["q"], q)] + gate
+        return [(n["q"], q), (n["k"], k), (n["v"], self.num_kv_heads * self.v_head_dim)] + gate
 
     def own_specs(self):
         n, specs = self.names, {}
@@ -276,6 +288,8 @@ class WindowAttention(ProjectedPart, Mixer):
         f32 = lambda name: tensors[name].to(device=rt.device, dtype=torch.float32).contiguous()
         if self.has_sink:
             self.sink = f32(self.names["sink"])
+        elif self.sink_score is not None:
+            self.sink = torch.full((self.num_heads * self.maps,), self.sink_score, device=rt.device, dtype=torch.float32)
         if self.sigmoid_weights:
             self.sigmoid_bias = f32(self.names["sigmoid_bias"])
         if self.maps == 2:
@@ -297,12 +311,14 @@ class WindowAttention(ProjectedPart, Mixer):
         write = self.own_kv and cache.write
         if self.by_head:
             coef, every = self.q_temperature or (0.0, 0)
+            extra = {"rotary": self.pos_enc.rotary()} if self.pos_enc is not None else {}
             ops.head_norm_kv_write(q, k, v, self.num_heads, self.num_kv_heads, self.head_dim, self.v_head_dim,
                                    self.q_norm_weight, self.k_norm_weight, self.qk_norm_eps or 1.0, ctx.positions,
                                    ctx.row_of_token, cache.k, cache.v, table, cache.page_size, write_kv=write,
-                                   norm=self.qk_norm_eps is not None, temp_coef=coef, temp_every=every, maps=self.maps)
+                                   norm=self.qk_norm_eps is not None, temp_coef=coef, temp_every=every, maps=self.maps,
+                                   **extra)
             ops.window_attention(q, act, self.num_heads, self.num_kv_heads, self.head_dim, self.v_head_dim, cache.k, cache.v,
-                                 table, cache.page_size, ctx, self.scale, self.window or 0, None, False, **self._weights_how())
+                                 table, cache.page_size, ctx, self.scale, self.window or 0, None, False, **self._weights_how(proj))
             return
         rotary = self.pos_enc.rotary() if self.pos_enc is not None else None
         vrot = self.value_pos_enc.rotary()[:2] if self.value_pos_enc is not None else None
@@ -314,9 +330,9 @@ class WindowAttention(ProjectedPart, Mixer):
                             write_kv=write, interleaved_values=self.interleaved_values, **extra)
         ops.window_attention(q, act, self.num_heads, self.num_kv_heads, self.head_dim, self.v_head_dim, cache.k, cache.v,
                              table, cache.page_size, ctx, self.scale, self.window or 0, vrot, self.interleaved_values,
-                             **self._weights_how())
+                             **self._weights_how(proj))
 
-    def _weights_how(self):
+    def _weights_how(self, proj):
         """What the attention kernels are told beside the sizes, the scale and the window."""
         how = {}
         if self.sink is not None:
@@ -329,6 +345,10 @@ class WindowAttention(ProjectedPart, Mixer):
             how["chunk"] = self.chunk
         if self.maps == 2:
             how["difference"] = (self.lam, 1.0 - self.difference, self.difference_eps)
+        if self.softcap:
+            how["softcap"] = self.softcap
+        if self.head_gate:
+            how["gate"] = proj[self.names["g"]]
         return how
 
 
@@ -351,14 +371,19 @@ class LatentAttention(ProjectedPart, Mixer):
     ``window``: a position sees itself and the ``window - 1`` before it (None: all); the cache gives back the
     pages the window has passed.  ``sink``: a learned number a head (tensor ``sink``) whose exponential joins
     the softmax's denominator; it has no key and no value and is not scaled.
+    ``q_rank``: the queries come from a latent of their own, ``W_q (normed W_dq x)`` with ``q_rank`` features between (tensors
+    ``dq``, ``dq.norm``, and ``uq`` in place of ``q``).  ``output_gate``: the heads' outputs side by side are multiplied,
+    feature by feature, by the sigmoid of one more projection of the input (tensor ``g``).
     Tensor names: ``q, dkv, dkv.norm, uk, uv, o, sink`` unless given."""
 
     is_mixer = True
 
     def __init__(self, hidden_size: int, num_heads: int, head_dim: int, rot_dim: int, v_head_dim: int, latent_dim: int,
                  scale: float, norm_eps: float, pos_enc: Optional[PositionEncoding] = None, interleaved: bool = True,
-                 names: Optional[Dict[str, str]] = None, window: Optional[int] = None, sink: bool = False):
+                 names: Optional[Dict[str, str]] = None, window: Optional[int] = None, sink: bool = False,
+                 q_rank: Optional[int] = None, output_gate: bool = False):
         self.hidden_size = int(hidden_size)
+        self.q_rank, self.output_gate = (int(q_rank) if q_rank else None), bool(output_gate)
         self.window = int(window) if window else None
         self.has_sink = bool(sink)
         self.sink = None
@@ -366,13 +391,20 @@ class LatentAttention(ProjectedPart, Mixer):
         self.v_head_dim, self.latent_dim = int(v_head_dim), int(latent_dim)
         self.scale, self.norm_eps = float(scale), float(norm_eps)
         self.pos_enc, self.interleaved = pos_enc, bool(interleaved)
-        self.names = {"q": "q", "down": "dkv", "norm": "dkv.norm", "uk": "uk", "uv": "uv", "o": "o", "sink": "sink"}
+        self.names = {"q": "q", "down": "dkv", "norm": "dkv.norm", "uk": "uk", "uv": "uv", "o": "o", "sink": "sink",
+                      "q_down": "dq", "q_norm": "dq.norm", "q_up": "uq", "gate": "g"}
         if names:
             self.names.update(names)
+        self.q_width = self.num_heads * (self.head_dim + self.rot_dim)
+        self.q_up = Linear(self.q_rank, self.q_width) if self.q_rank else None
 
     def in_projections(self):
         n = self.names
-        return [(n["q"], self.num_heads * (self.head_dim + self.rot_dim)), (n["down"], self.latent_dim + self.rot_dim)]
+        rows = [(n["q"], self.q_width) if self.q_rank is None else (n["q_down"], self.q_rank)]
+        rows.append((n["down"], self.latent_dim + self.rot_dim))
+        if self.output_gate:
+            rows.append((n["gate"], self.num_heads * self.v_head_dim))
+        return rows
 
     def out_projection(self):
         return (self.names["o"], self.num_heads * self.v_head_dim)
@@ -383,6 +415,8 @@ class LatentAttention(ProjectedPart, Mixer):
                  n["uv"]: ParamSpec((H * self.v_head_dim, R))}
         if self.has_sink:
             specs[n["sink"]] = ParamSpec((H,), mean=0.0, std=1.0)
+        if self.q_rank is not None:
+            specs[n["q_norm"]], specs[n["q_up"]] = ParamSpec((self.q_rank,), "norm"), ParamSpec((self.q_width, self.q_rank))
         return specs
 
     def cache_need(self):
@@ -397,7 +431,7 @@ class LatentAttention(ProjectedPart, Mixer):
 
     def arrange_in(self, name: str, w: torch.Tensor) -> torch.Tensor:
         d, r, R = self.head_dim, self.rot_dim, self.latent_dim
-        if name == self.names["q"]:
+        if name == self.names["q"] or name == self.names["q_up"]:
             heads = w.view(self.num_heads, d + r, w.shape[1])
             return torch.cat([torch.cat([h[:d], self._pairs_apart(h[d:])], dim=0) for h in heads], dim=0)
         if name == self.names["down"]:
@@ -418,22 +452,35 @@ class LatentAttention(ProjectedPart, Mixer):
         self.w_value = tensors[n["uv"]].to(device=rt.device, dtype=rt.dtype).contiguous().view(H, self.v_head_dim, R)
         if self.has_sink:
             self.sink = tensors[n["sink"]].to(device=rt.device, dtype=torch.float32).contiguous()
+        if self.q_rank is not None:
+            self.q_norm_weight = tensors[n["q_norm"]].to(device=rt.device, dtype=torch.float32).contiguous()
+            self.q_up.set_weight(self.arrange_in(n["q_up"], tensors[n["q_up"]].to(device=rt.device, dtype=rt.dtype)), rt)
 
     def core(self, ctx, proj, act, cache) -> None:
         ops, n, ws = self.rt.ops, self.names, ctx.workspace
         H, d, r, R = self.num_heads, self.head_dim, self.rot_dim, self.latent_dim
-        q, down = proj[n["q"]], proj[n["down"]]
-        T = q.shape[0]
+        down = proj[n["down"]]
+        T = down.shape[0]
         table = ctx.block_tables[cache.group]
         q_lat = ws.get("latent.q", T, H * (R + r), self.rt.dtype)
         rotary = self.pos_enc.rotary() if self.pos_enc is not None else None
-        ops.latent_kv_write(q, down, q_lat, H, d, r, R, self.norm_weight, self.norm_eps, rotary, ctx.positions,
-                            ctx.row_of_token, cache.k, cache.v, table, cache.page_size, write_kv=cache.write)
-        ops.head_linear(q, d + r, self.w_absorb, q_lat, R + r)
+        kv = (self.norm_weight, self.norm_eps, rotary, ctx.positions, ctx.row_of_token, cache.k, cache.v, table, cache.page_size)
+        if self.q_rank is None:
+            q = proj[n["q"]]
+            ops.latent_kv_write(q, down, q_lat, H, d, r, R, *kv, write_kv=cache.write)
+            ops.head_linear(q, d + r, self.w_absorb, q_lat, R + r)
+        else:
+            normed = ws.get("latent.q_latent", T, self.q_rank, self.rt.dtype)
+            ops.latent_kv_write(None, down, None, H, d, r, R, *kv, write_kv=cache.write,
+                                query_latent=(proj[n["q_down"]], self.q_norm_weight, normed))
+            q = ws.get("latent.q_heads", T, self.q_width, self.rt.dtype)
+            self.q_up.forward(normed, q)
+            ops.head_linear(q, d + r, self.w_absorb, q_lat, R + r, tail=r, rotary=rotary, positions=ctx.positions)
+        gate = {"gate": proj[n["gate"]]} if self.output_gate else {}
         lat = ws.get("latent.sum", T, H * R, self.rt.dtype)
         for h0 in range(0, H, self.heads_a_call):
             n = min(self.heads_a_call, H - h0)
             ops.window_attention(q_lat[:, h0 * (R + r):(h0 + n) * (R + r)], lat[:, h0 * R:(h0 + n) * R], n, 1, R + r, R,
                                  cache.k, cache.v, table, cache.page_size, ctx, self.scale, self.window or 0, None, False,
                                  sink=self.sink[h0:h0 + n] if self.sink is not None else None)
-        ops.head_linear(lat, R, self.w_value, act, self.v_head_dim)
+        ops.head_linear(lat, R, self.w_value, act, self.v_head_dim, **gate)

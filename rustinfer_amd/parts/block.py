@@ -479,6 +479,155 @@ class SandwichBlock(Part):
         self._run_half(ctx, hidden, self.halves[0], cache, None, only_state=True)
 
 
+class HyperConnection(Part):
+    """How one sub-layer reads and writes a residual stream of ``n`` rows a token: it reads ``sum_s in[s] x_s`` (behind its
+    norm), and with its result ``y`` the rows become ``x'_t = sum_s mix[s, t] x_s + out[t] y``, all at once from the old ones.
+    Tensors ``in [n]``, ``out [n]``, ``mix [n, n]`` (from, to), kept in 32-bit."""
+
+    def __init__(self, streams: int):
+        self.streams = int(streams)
+
+    def param_specs(self) -> Dict[str, ParamSpec]:
+        n = self.streams
+        near = lambda shape, mean: (lambda g, s, device: mean.to(device) + 0.1 * torch.randn(shape, generator=g, device=device))
+        return {"in": ParamSpec((n,), init=near((n,), torch.full((n,), 1.0 / n))), "out": ParamSpec((n,), mean=1.0, std=0.1),
+                "mix": ParamSpec((n, n), init=near((n, n), torch.eye(n)))}
+
+    def load(self, tensors, rt: Runtime) -> None:
+        self.rt = rt
+        f32 = lambda name: tensors[name].to(device=rt.device, dtype=torch.float32).contiguous()
+        self.in_w, self.out_w, self.mix = f32("in"), f32("out"), f32("mix")
+
+
+class PendingStreams:
+    """``Hidden.pending`` of a model whose residual has several rows a token: the rows ``streams [T, n, d]`` (None: all of
+    them are ``Hidden.x`` still), what the last sub-layer returned, and the ``HyperConnection`` by which it joins them."""
+
+    __slots__ = ("streams", "delta", "connection")
+
+    def __init__(self, streams, delta, connection: HyperConnection):
+        self.streams, self.delta, self.connection = streams, delta, connection
+
+    def enter(self, ops, x, in_w, norm: Norm, act, streams_out=None, rows=None):
+        """Join the delta to the rows and leave ``norm(sum_t in_w[t] x'_t)`` in ``act``."""
+        c = self.connection
+        ops.hyper_streams(x if self.streams is None else self.streams, c.streams, in_w, norm.weight, norm.eps, act, delta=self.delta,
+                          mix=c.mix, out_w=c.out_w, bias=getattr(norm, "bias", None), streams_out=streams_out, rows=rows,
+                          centered=getattr(norm, "layer_norm", False))
+
+
+class StreamsNorm(Norm):
+    """The norm behind the last block of a model of several residual rows: ``norm`` (a ``LayerNorm``, or an ``RMSNorm`` with
+    a 32-bit weight) of the rows' sum, in the pass that joins the last sub-layer's result to them."""
+
+    cuts_rows = False
+    plain_rms = False
+
+    def __init__(self, norm: Norm, streams: int):
+        self.norm, self.streams = norm, int(streams)
+
+    def param_specs(self) -> Dict[str, ParamSpec]:
+        return self.norm.param_specs()
+
+    def load(self, tensors, rt: Runtime) -> None:
+        self.rt = rt
+        self.norm.load(tensors, rt)
+        self.ones = torch.ones(self.streams, device=rt.device, dtype=torch.float32)
+
+    def forward(self, ctx, x, delta, out, rows=None, x_rows=None):
+        if not isinstance(delta, PendingStreams):
+            raise RuntimeError("the norm over several residual rows follows a block that keeps them")
+        delta.enter(self.rt.ops, x, self.ones, self.norm, out, rows=rows)
+        return out
+
+
+class HyperConnectedBlock(Part):
+    """A pre-norm block on a residual of ``streams`` rows a token: the mixer and the feed-forward (which may be absent)
+    each read and write the rows through a ``HyperConnection``.  The norms are ``LayerNorm`` (or ``RMSNorm`` with a 32-bit
+    weight).  Joining a sub-layer's result to the rows, the weighted sum the next one reads and its norm are one kernel;
+    a result stays pending until then (``PendingStreams``), so the streams are read and written once a sub-layer."""
+
+    takes_follow = False
+
+    def __init__(self, hidden_size: int, streams: int, mixer_norm: Norm, mixer: Mixer, ffn_norm: Optional[Norm] = None,
+                 ffn: Optional[FeedForward] = None, names: Optional[Dict[str, str]] = None):
+        if mixer is None or mixer_norm is None or (ffn is None) != (ffn_norm is None):
+            raise ValueError("a block needs a mixer, and a sub-layer and its norm come together")
+        self.hidden_size, self.streams = int(hidden_size), int(streams)
+        self.mixer_norm, self.mixer, self.ffn_norm, self.ffn = mixer_norm, mixer, ffn_norm, ffn
+        self.mixer_connection = HyperConnection(streams)
+        self.ffn_connection = HyperConnection(streams) if ffn is not None else None
+        self.names = {"mixer_norm": "norm1", "mixer": "mix", "mixer_connection": "hc1",
+                      "ffn_norm": "norm2", "ffn": "mlp", "ffn_connection": "hc2"}
+        if names:
+            self.names.update(names)
+
+    def _children(self):
+        for key in ("mixer_norm", "mixer_connection", "mixer", "ffn_norm", "ffn_connection", "ffn"):
+            part = getattr(self, key)
+            if part is not None:
+                yield self.names[key], part
+
+    def param_specs(self) -> Dict[str, ParamSpec]:
+        specs = {}
+        for prefix, part in self._children():
+            for name, spec in part.param_specs().items():
+                specs[join_name(prefix, name)] = spec
+        return specs
+
+    def load(self, tensors, rt: Runtime) -> None:
+        self.rt = rt
+        for prefix, part in self._children():
+            part.load(narrow_tensors(tensors, prefix), rt)
+        for norm in (self.mixer_norm, self.ffn_norm):
+            if norm is not None and norm.weight.dtype != torch.float32:
+                raise RuntimeError("the norms of a block on several residual rows keep their weights in 32-bit (weight_32bit=True)")
+
+    def cache_need(self):
+        return self.mixer.cache_need()
+
+    @property
+    def graph_safe(self) -> bool:
+        return all(getattr(part, "graph_safe", True) for _, part in self._children())
+
+    def can_cut_rows(self) -> bool:
+        return self.ffn is not None
+
+    def entry(self):
+        return (self.mixer_norm, None)           # nobody else can prepare what this block reads
+
+    def _enter(self, ctx, hidden: Hidden, connection: HyperConnection, norm: Norm, rows=None):
+        """What the sub-layer behind ``norm`` reads; the rows' new values are kept for the next sub-layer.  Returns (those
+        rows or None, the input)."""
+        ops, ws, d, n = self.rt.ops, ctx.workspace, self.hidden_size, self.streams
+        T = hidden.x.shape[0] if rows is None else rows.numel()
+        act = ws.get("block.normed" if rows is None else "block.normed_rows", T, d, self.rt.dtype)
+        p = hidden.pending
+        if p is None:                            # the first sub-layer: every row is the embedded one still
+            ops.hyper_streams(hidden.x, n, connection.in_w, norm.weight, norm.eps, act, bias=getattr(norm, "bias", None),
+                              centered=getattr(norm, "layer_norm", False))
+            return None, act
+        kept = ws.get("block.streams" if rows is None else "block.streams_rows", T, n * d, torch.float32).view(T, n, d)
+        p.enter(ops, hidden.x, connection.in_w, norm, act, streams_out=kept, rows=rows)
+        return kept, act
+
+    def forward(self, ctx, hidden: Hidden, cache, out_rows: Optional[torch.Tensor] = None, follow=None) -> None:
+        """``out_rows``: nothing after this block needs the other rows of the step; the feed-forward runs on those alone,
+        and the pending streams are theirs."""
+        streams, inp = self._enter(ctx, hidden, self.mixer_connection, self.mixer_norm)
+        hidden.pending, hidden.deferred = PendingStreams(streams, self.mixer.forward(ctx, inp, cache), self.mixer_connection), None
+        if self.ffn is not None:
+            streams, inp = self._enter(ctx, hidden, self.ffn_connection, self.ffn_norm, rows=out_rows)
+            hidden.pending = PendingStreams(streams, self.ffn.forward(ctx, inp), self.ffn_connection)
+
+    def update_cache_only(self, ctx, hidden: Hidden, cache) -> None:
+        """The last block of a step whose logits nobody wants: the mixer alone runs, for what it leaves in its cache or
+        state; ``hidden`` is not meaningful afterwards."""
+        _, inp = self._enter(ctx, hidden, self.mixer_connection, self.mixer_norm)
+        update = getattr(self.mixer, "update_cache", None)
+        (update or self.mixer.forward)(ctx, inp, cache)
+
+
 class TwoMixers(Mixer):
     """A mixer made of two that read the same rows side by side: ``left_scale * left(h) + right_scale * right(h)``.
     Both halves are ``ProjectedPart``: their input projections are one product, their output projections one

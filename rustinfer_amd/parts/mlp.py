@@ -162,6 +162,9 @@ class MoEFeedForward(FeedForward):
     ``limit``: every expert's activation is the clipped one, ``g' sigmoid(slope g') (u' + shift)`` with
     ``g' = min(g, limit)`` and ``u' = clamp(u, -limit, limit)`` (``shared_limit``: the shared expert's limit).
     ``weigh_input``: an expert runs on its token's row multiplied by the weight, instead of its output being multiplied.
+    ``score = "chosen_softmax"``: the ``top`` largest logits are chosen, and the weights are the softmax over those alone.
+    ``router_bias``: a number an expert (tensor ``router.b``) is added to its logits, in 32-bit.
+    ``gated = False``: no gate matrices (the shared expert has none either): an expert is ``W_down relu(W_up x)^2``.
     Tensor names: ``router``, ``e<i>.gate``, ``e<i>.up``, ``e<i>.down``."""
 
     # up to this many tokens in a step every block of the activation kernel makes its token's weights
@@ -172,11 +175,14 @@ class MoEFeedForward(FeedForward):
     def __init__(self, hidden_size: int, expert_size: int, experts: int, top: int, renormalize: bool = False,
                  score: str = "softmax", norm_eps: float = 0.0, scale: float = 1.0, shared_size: int = 0,
                  shared_gate: bool = False, limit: Optional[float] = None, shared_limit: Optional[float] = None,
-                 slope: float = 1.702, shift: float = 1.0, weigh_input: bool = False):
+                 slope: float = 1.702, shift: float = 1.0, weigh_input: bool = False, gated: bool = True,
+                 router_bias: bool = False):
         if not (0 < top <= experts):
             raise ValueError(f"top {top} of {experts} experts")
-        if score not in ("softmax", "sigmoid"):
-            raise ValueError(f"a router scores with 'softmax' or 'sigmoid', got {score!r}")
+        if score not in ("softmax", "sigmoid", "chosen_softmax"):
+            raise ValueError(f"a router scores with 'softmax', 'sigmoid' or 'chosen_softmax', got {score!r}")
+        if not gated and limit is not None:
+            raise ValueError("the clipped activation belongs to experts with a gate")
         self.hidden_size, self.expert_size = int(hidden_size), int(expert_size)
         self.experts, self.top, self.renormalize = int(experts), int(top), bool(renormalize)
         self.score, self.norm_eps, self.scale, self.shared_size = score, float(norm_eps), float(scale), int(shared_size)
@@ -187,22 +193,27 @@ class MoEFeedForward(FeedForward):
         self.shared_limit = float(shared_limit) if shared_limit is not None else self.limit
         self.slope, self.shift = float(slope), float(shift)
         self.clip = None
-        self.plain = score == "softmax" and self.scale == 1.0 and self.norm_eps == 0.0 and self.shared_size == 0
+        self.gated, self.router_bias = bool(gated), bool(router_bias)
+        self.bias = None
+        self.plain = self.gated and not self.router_bias and score == "softmax" and self.scale == 1.0 and self.norm_eps == 0.0 and self.shared_size == 0
         # columns of the activations: the experts', the shared expert's, zeros up to a multiple of eight
         self.act_width = (self.experts * self.expert_size + self.shared_size + 7) // 8 * 8
         self.logits_width = self.experts + int(self.shared_gate)
         self.router = Linear(self.hidden_size, self.logits_width)
-        self.gate_up = Linear(self.hidden_size, 2 * self.experts * self.expert_size + 2 * self.shared_size)
+        self.gate_up_width = (2 if self.gated else 1) * (self.experts * self.expert_size + self.shared_size)
+        self.gate_up = Linear(self.hidden_size, self.gate_up_width)
         self.down = Linear(self.act_width, self.hidden_size)
 
     def param_specs(self) -> Dict[str, ParamSpec]:
         h, f = self.hidden_size, self.expert_size
         specs = {"router": ParamSpec((self.experts, h))}
-        for e in range(self.experts):
-            specs[f"e{e}.gate"], specs[f"e{e}.up"], specs[f"e{e}.down"] = ParamSpec((f, h)), ParamSpec((f, h)), ParamSpec((h, f))
-        if self.shared_size:
-            s = self.shared_size
-            specs["shared.gate"], specs["shared.up"], specs["shared.down"] = ParamSpec((s, h)), ParamSpec((s, h)), ParamSpec((h, s))
+        if self.router_bias:
+            specs["router.b"] = ParamSpec((self.experts,), mean=0.0, std=0.5)
+        groups = [(f"e{e}", f) for e in range(self.experts)] + ([("shared", self.shared_size)] if self.shared_size else [])
+        for name, size in groups:
+            if self.gated:
+                specs[name + ".gate"] = ParamSpec((size, h))
+            specs[name + ".up"], specs[name + ".down"] = ParamSpec((size, h)), ParamSpec((h, size))
         if self.shared_gate:
             specs["shared.sg"] = ParamSpec((1, h))
         return specs
@@ -216,10 +227,13 @@ class MoEFeedForward(FeedForward):
         self.router.set_weight(router, rt, tile=False)
         if self.limit is not None:
             self.clip = rt.ops.ClippedGate(self.limit, self.shared_limit, self.slope, self.shift)
-        rows = [to(f"e{e}.{n}") for e in range(self.experts) for n in ("gate", "up")]
+        if self.router_bias:
+            self.bias = tensors["router.b"].to(device=rt.device, dtype=torch.float32).contiguous()
+        ins = ("gate", "up") if self.gated else ("up",)
+        rows = [to(f"e{e}.{n}") for e in range(self.experts) for n in ins]
         cols = [to(f"e{e}.down") for e in range(self.experts)]
         if self.shared_size:
-            rows += [to("shared.gate"), to("shared.up")]
+            rows += [to(f"shared.{n}") for n in ins]
             cols.append(to("shared.down"))
         pad = self.act_width - self.experts * self.expert_size - self.shared_size
         if pad:
@@ -232,7 +246,7 @@ class MoEFeedForward(FeedForward):
         T, E, F = normed.shape[0], self.experts, self.expert_size
         logits = ws.get("moe.logits", T, self.logits_width, torch.float32)
         self.router.forward(normed, logits)
-        gate_up = ws.get("moe.gate_up", T, 2 * E * F + 2 * self.shared_size, self.rt.dtype)
+        gate_up = ws.get("moe.gate_up", T, self.gate_up_width, self.rt.dtype)
         self.gate_up.forward(normed, gate_up)
         act = ws.get("moe.act", T, self.act_width, self.rt.dtype)
         how = {} if self.plain else {"score": self.score, "norm_eps": self.norm_eps, "scale": self.scale}
@@ -244,6 +258,10 @@ class MoEFeedForward(FeedForward):
             shared["clip"] = self.clip
         if self.weigh_input:
             shared["weigh_input"] = True
+        if not self.gated:
+            shared["gated"] = False
+        if self.bias is not None:
+            how["bias"] = self.bias
         if T <= self.ROUTE_ON_THE_WAY_ROWS:
             ops.moe_swiglu_routed(gate_up, logits, act, E, F, self.top, self.renormalize, **how, **shared)
         else:

@@ -9,7 +9,7 @@ in 32-bit, so the sum is rounded once, into ``out``.
 """
 from __future__ import annotations
 
-from typing import Dict
+from typing import Dict, Optional
 
 import torch
 
@@ -99,24 +99,28 @@ class OutputRMSNorm(Norm):
 class LayerNorm(Norm):
     """``(x - mean) / sqrt(var + eps) * w + b`` over each row, the variance being the mean of the squared
     deviations; 32-bit arithmetic, weight and bias kept in 32-bit.  Tensors: the weight under
-    ``weight_name`` ("" where it carries the norm's own name), the bias under that name + ``bias_suffix``."""
+    ``weight_name`` ("" where it carries the norm's own name), the bias under ``bias_name`` (None: no bias)."""
 
     cuts_rows = False
     plain_rms = False
     layer_norm = True          # a block may make this norm's output in the pass that last changes the stream
 
-    def __init__(self, dim: int, eps: float, weight_name: str = "weight", bias_name: str = "bias"):
+    def __init__(self, dim: int, eps: float, weight_name: str = "weight", bias_name: Optional[str] = "bias"):
         self.dim, self.eps = int(dim), float(eps)
         self.weight_name, self.bias_name = weight_name, bias_name
         self.weight = self.bias = None
 
     def param_specs(self) -> Dict[str, ParamSpec]:
-        return {self.weight_name: ParamSpec((self.dim,), "norm"), self.bias_name: ParamSpec((self.dim,), mean=0.0, std=0.1)}
+        specs = {self.weight_name: ParamSpec((self.dim,), "norm")}
+        if self.bias_name is not None:
+            specs[self.bias_name] = ParamSpec((self.dim,), mean=0.0, std=0.1)
+        return specs
 
     def load(self, tensors, rt: Runtime) -> None:
         self.rt = rt
         f32 = lambda name: tensors[name].to(device=rt.device, dtype=torch.float32).contiguous()
-        self.weight, self.bias = f32(self.weight_name), f32(self.bias_name)
+        self.weight = f32(self.weight_name)
+        self.bias = f32(self.bias_name) if self.bias_name is not None else None
 
     def forward(self, ctx, x, delta, out, rows=None, x_rows=None):
         if delta is not None or x_rows is not None:
