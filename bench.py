@@ -640,15 +640,62 @@ class ZotonexBench(TedelixBench):
         self.attn_flops_per_key = sum(2.0 * 2 * l.mixer.heads * (l.mixer.dim + l.mixer.vdim) for l in cfg.layers)
 
 
+# Sibodra at the layer sizes of the Llama shapes: the same width, number of layers and heads; four residual rows a token;
+# soft-capped attention and attention through latents take turns (Belorax's latent and rotated part, queries from a latent
+# of half the width); two layers with gated feed-forwards of the shape's width, two with eight experts and a shared one without gates,
+# 3/8 of it wide, so that eight of them have the weights of Belorax's eight.
+SIBODRA_PATTERN = ("attention", "latent_attention")
+
+
+def sibodra_config(shape_name, layers=0, streams=4):
+    s = SHAPES[shape_name]
+    H, G, hd, W, ff = s["num_attention_heads"], s["num_key_value_heads"], s["head_dim"], s["hidden_size"], s["intermediate_size"]
+    out = []
+    for i in range(layers or s["num_hidden_layers"]):
+        kind = SIBODRA_PATTERN[i % len(SIBODRA_PATTERN)]
+        if kind == "attention":
+            mixer = dict(heads=H, kv_heads=G, dim=hd, vdim=hd, scale=hd ** -0.5, softcap=30.0,
+                         rot=dict(base=10000.0, dims=hd // 2, scaling=dict(factor=4.0, low=1.0, high=4.0, original=1024)))
+        else:
+            r = hd // 2
+            mixer = dict(heads=H, dim=hd, rot_dim=r, vdim=hd, q_rank=W // 2, kv_rank=256 - r, scale=(hd + r) ** -0.5, rot=dict(base=10000.0, dims=r))
+        e = 3 * ff // 8
+        mlp = dict(kind="dense", ff=ff) if i // 2 % 2 == 0 else dict(kind="moe", expert=dict(ff=e), shared=dict(ff=e), router=dict(experts=8, top=2))
+        out.append(dict(type=kind, mixer=mixer, mlp=mlp))
+    return dict(architecture="Sibodra", vocab=s["vocab_size"], width=W, streams=streams, norm=dict(eps=1e-5), logit_softcap=30.0, layers=out)
+
+
+class SibodraBench(TedelixBench):
+    """The same measurements on a Sibodra model of a Llama shape's sizes."""
+
+    def design_config(self, shape_name, args):
+        self.window = 1 << 30                         # no window: a request reads all its keys
+        return sibodra_config(shape_name, args.layers)
+
+    def account(self, cfg, el):
+        self.window_kv_bytes = self.state_bytes = 0
+        self.attn_flops_per_key = self.scan_flops_per_token = 0
+        for layer in cfg.layers:
+            m = layer.mixer
+            if layer.type == "attention":
+                self.window_kv_bytes += m.kv_heads * (m.dim + m.vdim) * el
+                self.attn_flops_per_key += 2.0 * m.heads * (m.dim + m.vdim)
+            else:
+                self.window_kv_bytes += (2 * m.kv_rank + m.rot_dim) * el            # the latent lies there as key and as value
+                self.attn_flops_per_key += 2.0 * m.heads * (2 * m.kv_rank + m.rot_dim)
+
+
 DESIGNS = {"tedelix": (TedelixBench, "llama", TEDELIX_PATTERN), "belorax": (BeloraxBench, "tedelix", BELORAX_PATTERN),
            "pilavik": (PilavikBench, "belorax", PILAVIK_PATTERN), "debuzen": (DebuzenBench, "pilavik", DEBUZEN_PATTERN),
-           "zotonex": (ZotonexBench, "belorax", ("attention", "attention on a borrowed cache"))}
+           "zotonex": (ZotonexBench, "belorax", ("attention", "attention on a borrowed cache")),
+           "sibodra": (SibodraBench, "belorax", SIBODRA_PATTERN)}
 
 
 def design_record(args, peaks):
-    """``--design tedelix|belorax|pilavik|debuzen|zotonex``: decode at the main batch and prefill of 2,048 tokens for
+    """``--design tedelix|belorax|pilavik|debuzen|zotonex|sibodra``: decode at the main batch and prefill of 2,048 tokens for
     models of that design at the sizes of ``--design-shapes``, each beside the closest other design at the same
-    sizes (Tedelix beside Llama, Belorax beside Tedelix, Pilavik beside Belorax, Debuzen beside Pilavik, Zotonex beside Belorax)."""
+    sizes (Tedelix beside Llama, Belorax beside Tedelix, Pilavik beside Belorax, Debuzen beside Pilavik, Zotonex and
+    Sibodra beside Belorax)."""
     design_cls, beside, pattern = DESIGNS[args.design]
     others = {"llama": Bench, "tedelix": TedelixBench, "belorax": BeloraxBench, "pilavik": PilavikBench}
     out = {"metric": "decode tok/s at batch %d and prefill tok/s at 2,048 tokens: %s beside %s at equal layer sizes" % (args.batch, args.design, beside),
@@ -751,10 +798,10 @@ def main() -> int:
                     help="only time the sampling kernels on 1, 8 and 64 rows of the shape's vocabulary")
     ap.add_argument("--no-gemm-tune", action="store_true",
                     help="keep the GEMM library's own choice of kernel for the prompt's products")
-    ap.add_argument("--design", default="llama", choices=["llama", "tedelix", "belorax", "pilavik", "debuzen", "zotonex"],
-                    help="tedelix, belorax, pilavik, debuzen, zotonex: only decode and prefill of models of that design at the sizes of "
+    ap.add_argument("--design", default="llama", choices=["llama", "tedelix", "belorax", "pilavik", "debuzen", "zotonex", "sibodra"],
+                    help="tedelix, belorax, pilavik, debuzen, zotonex, sibodra: only decode and prefill of models of that design at the sizes of "
                          "--design-shapes, each beside the closest other design at the same sizes (Tedelix beside Llama, "
-                         "Belorax beside Tedelix, Pilavik beside Belorax, Debuzen beside Pilavik, Zotonex beside Belorax; the default workload is not run)")
+                         "Belorax beside Tedelix, Pilavik beside Belorax, Debuzen beside Pilavik, Zotonex and Sibodra beside Belorax; the default workload is not run)")
     ap.add_argument("--design-shapes", default="1b,3b", help="shapes for --design other than llama, with commas between them")
     args = ap.parse_args()
     if args.gpus != 1:

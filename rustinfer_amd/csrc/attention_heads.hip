@@ -80,10 +80,95 @@ __global__ __launch_bounds__(256) void head_norm_kv_write_kernel(
     }
 }
 
+// The same with eight features a lane (16 bytes of bfloat16 a load): dk, the turned half and every row stride multiples of
+// eight.  LPH lanes, a power of two that holds dk / 8, share a head; a block's 256 / LPH heads go side by side, so a token's
+// heads are read at once instead of one behind the other.
+template <typename T, int LPH>
+__global__ __launch_bounds__(256) void head_norm_kv_write_vec_kernel(
+        T* __restrict__ q, int q_stride, const T* __restrict__ k, int k_stride, const T* __restrict__ v, int v_stride,
+        int H, int Hkv, int dk, int dv, const float* __restrict__ qw, const float* __restrict__ kw, int do_norm, float eps,
+        float temp_coef, int temp_every, const int* __restrict__ positions, const int* __restrict__ row_of_token,
+        T* __restrict__ kc, T* __restrict__ vc, const int* __restrict__ table, int max_blocks, int page, int write_kv, int maps,
+        int rot, const float* __restrict__ cos_t, const float* __restrict__ sin_t) {
+    using L = VecLoad<4>;
+    const int t = blockIdx.x;
+    const int b = row_of_token[t];
+    if (b < 0) return;                       // padding token
+    const int pos = positions[t];
+    const int Hq = H * maps, Hk = Hkv * maps;
+    int blk = -1;
+    if (write_kv) blk = table[(size_t)b * max_blocks + pos / page];
+    const int slot = pos % page;
+    const float temp = temp_every > 0 ? 1.f + temp_coef * logf((float)((pos + 1) / temp_every) + 1.f) : 1.f;
+    const int units = Hq + (blk >= 0 ? Hk : 0);
+    const int l = threadIdx.x % LPH, i = 8 * l, half = rot >> 1;
+    const bool mine = i < dk, low = i < half;
+    const int partner = low ? l + half / 8 : l - half / 8;         // (used where i < rot)
+    float c[8], s[8];
+    if (mine && i < rot) {
+        const size_t at = (size_t)pos * half + (low ? i : i - half);
+#pragma unroll
+        for (int e = 0; e < 8; e += 4) { L::ld(cos_t + at + e, c + e); L::ld(sin_t + at + e, s + e); }
+    }
+    constexpr int HPB = 256 / LPH;
+    // (every lane of a wave goes round equally often: the shuffles below are met by all)
+    for (int u0 = blockIdx.y * HPB; u0 < units; u0 += HPB * gridDim.y) {
+        const int u = u0 + threadIdx.x / LPH;
+        const bool on = mine && u < units, is_q = u < Hq;
+        const int g = is_q ? 0 : u - Hq;
+        float x[8];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[e] = 0.f;
+        if (on) {
+            const T* src = is_q ? q + (size_t)t * q_stride + u * dk + i : k + (size_t)t * k_stride + g * dk + i;
+#pragma unroll
+            for (int e = 0; e < 8; e += 4) L::ld(src + e, x + e);
+        }
+        float f = is_q ? temp : 1.f;
+        if (do_norm) {
+            float ss = 0.f;
+#pragma unroll
+            for (int e = 0; e < 8; ++e) ss = fmaf(x[e], x[e], ss);
+#pragma unroll
+            for (int o = LPH / 2; o > 0; o >>= 1) ss += __shfl_xor(ss, o, LPH);
+            f *= 1.f / sqrtf(ss / (float)dk + eps);
+        }
+        const float* w = is_q ? qw : kw;
+        float wv[8];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) wv[e] = 1.f;
+        if (on && w) {
+#pragma unroll
+            for (int e = 0; e < 8; e += 4) L::ld(w + i + e, wv + e);
+        }
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[e] = x[e] * f * wv[e];
+        if (rot > 0) {                       // (uniform)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                const float y = __shfl(x[e], partner & (LPH - 1), LPH);
+                if (i < rot) x[e] = low ? x[e] * c[e] - y * s[e] : x[e] * c[e] + y * s[e];
+            }
+        }
+        if (on) {
+            T* dst = is_q ? q + (size_t)t * q_stride + u * dk + i : kc + (((size_t)blk * Hkv + g / maps) * page + slot) * (maps * dk) + g % maps * dk + i;
+#pragma unroll
+            for (int e = 0; e < 8; e += 4) L::st(dst + e, x + e);
+        }
+    }
+    if (blk < 0) return;
+    const T* vrow = v + (size_t)t * v_stride;
+    for (int idx = blockIdx.y * 256 + threadIdx.x; idx < Hkv * dv; idx += 256 * gridDim.y) {
+        const int g = idx / dv, dd = idx - g * dv;
+        vc[(((size_t)blk * Hkv + g) * dv + dd) * page + slot] = vrow[idx];
+    }
+}
+
 // ---------------------------------------------------------------------------
 // One block a token.  q [T][H (d + r)]: a head's unrotated features, then its r rotated ones, of which
 // the first `rot` are turned (feature i with i + rot/2).  down [T][R + r].  q_abs [T][H (R + r)].
-// q null: the heads' queries are not there yet.  ql [T][Rq] (or null): the queries' latent, normed into ql_out [T][Rq].
+// q null: the heads' queries are not there yet.  ql [T][Rq] (or null): the queries' latent, normed into ql_out [T][Rq] by a
+// second block a token (blockIdx.y = 1).
 // ---------------------------------------------------------------------------
 template <typename T>
 __global__ __launch_bounds__(256) void latent_kv_write_kernel(
@@ -107,6 +192,15 @@ __global__ __launch_bounds__(256) void latent_kv_write_kernel(
         if (rotate && j < rot) return ld_f32(part + j) * cs[j - half] + ld_f32(part + j - half) * sn[j - half];
         return ld_f32(part + j);
     };
+    if (blockIdx.y == 1) {
+        const T* row = ql + (size_t)t * ql_stride;
+        float ss = 0.f;
+        for (int i = threadIdx.x; i < Rq; i += 256) { const float x = ld_f32(row + i); ss = fmaf(x, x, ss); }
+        ss = block_sum(ss, red);
+        const float rs = 1.f / sqrtf(ss / (float)Rq + eps);
+        for (int i = threadIdx.x; i < Rq; i += 256) st_f32(ql_out + (size_t)t * qo_stride + i, ld_f32(row + i) * rs * (qlw ? qlw[i] : 1.f));
+        return;
+    }
     if (q) {
         const T* qrow = q + (size_t)t * q_stride;
         T* qa = q_abs + (size_t)t * qa_stride;
@@ -114,14 +208,6 @@ __global__ __launch_bounds__(256) void latent_kv_write_kernel(
             const int h = idx / r, j = idx - h * r;
             st_f32(qa + h * (R + r) + R + j, turned(qrow + h * (d + r) + d, j));
         }
-    }
-    if (ql) {
-        const T* row = ql + (size_t)t * ql_stride;
-        float ss = 0.f;
-        for (int i = threadIdx.x; i < Rq; i += 256) { const float x = ld_f32(row + i); ss = fmaf(x, x, ss); }
-        ss = block_sum(ss, red);
-        const float rs = 1.f / sqrtf(ss / (float)Rq + eps);
-        for (int i = threadIdx.x; i < Rq; i += 256) st_f32(ql_out + (size_t)t * qo_stride + i, ld_f32(row + i) * rs * (qlw ? qlw[i] : 1.f));
     }
     if (!write_kv) return;
     const int blk = table[(size_t)b * max_blocks + pos / page];
@@ -242,7 +328,9 @@ __device__ __forceinline__ void hl_ld16(const bf16_t* p, float* f) {
     f[6] = __uint_as_float(v.w << 16); f[7] = __uint_as_float(v.w & 0xffff0000u);
 }
 
-template <typename T, bool VEC>
+// TT: the tokens a lane asks for at once (a step of fewer repeats its last one and drops the result): with a
+// bound in the loop instead every load would wait for the one before it.
+template <typename T, bool VEC, int TT>
 __global__ __launch_bounds__(256) void head_linear_few_kernel(
         const T* __restrict__ x, int x_stride, int x_head, const T* __restrict__ w, T* __restrict__ out, int out_stride,
         int out_head, int Tn, int N, int K, HeadExtra<T> extra) {
@@ -259,29 +347,91 @@ __global__ __launch_bounds__(256) void head_linear_few_kernel(
     const bool live = n < N;
     const T* wr = w + ((size_t)h * N + (live ? n : 0)) * K;
     const T* xh = x + (size_t)h * x_head;
-    float acc[HLF_T];
+    float acc[TT];
 #pragma unroll
-    for (int t = 0; t < HLF_T; ++t) acc[t] = 0.f;
+    for (int t = 0; t < TT; ++t) acc[t] = 0.f;
     for (int k = part * VL; k < K; k += 8 * VL) {
-        float wv[VL];
+        float wv[VL], xv[TT][VL];
         if (VEC) hl_ld16(wr + k, wv); else wv[0] = ld_f32(wr + k);
 #pragma unroll
-        for (int t = 0; t < HLF_T; ++t) {
-            if (t >= Tn) break;
-            float xv[VL];
-            if (VEC) hl_ld16(xh + (size_t)t * x_stride + k, xv); else xv[0] = ld_f32(xh + (size_t)t * x_stride + k);
-#pragma unroll
-            for (int u = 0; u < VL; ++u) acc[t] = fmaf(xv[u], wv[u], acc[t]);
+        for (int t = 0; t < TT; ++t) {
+            const T* row = xh + (size_t)min(t, Tn - 1) * x_stride + k;
+            if (VEC) hl_ld16(row, xv[t]); else xv[t][0] = ld_f32(row);
         }
-    }
 #pragma unroll
-    for (int t = 0; t < HLF_T; ++t) {
-        if (t >= Tn) break;
+        for (int t = 0; t < TT; ++t)
+#pragma unroll
+            for (int u = 0; u < VL; ++u) acc[t] = fmaf(xv[t][u], wv[u], acc[t]);
+    }
+    // all eight lanes have every token's sum; lane `part` writes the tokens part, part + 8
+    float keep[(TT + 7) / 8];
+#pragma unroll
+    for (int t = 0; t < TT; ++t) {
         float v = acc[t];
 #pragma unroll
         for (int o = 4; o > 0; o >>= 1) v += __shfl_xor(v, o, 8);
-        if (part == 0 && live) st_f32(out + (size_t)t * out_stride + h * out_head + n, extra.gated(v, t, h * N + n));
+        if ((t & 7) == part) keep[t >> 3] = v;
     }
+#pragma unroll
+    for (int j = 0; j < (TT + 7) / 8; ++j) {
+        const int t = part + 8 * j;
+        if (t < TT && t < Tn && live) st_f32(out + (size_t)t * out_stride + h * out_head + n, extra.gated(keep[j], t, h * N + n));
+    }
+}
+
+// The same product of many bfloat16 tokens on the matrix instructions (v_mfma_f32_32x32x16_bf16, 32-bit sums): a wave owns
+// 32 tokens and 64 outputs of one head, both operands straight from memory, 16 bytes a lane.  K and the row strides
+// multiples of eight; wide: the outputs may be written four at a time.
+typedef __bf16 hl_bf16x8_t __attribute__((ext_vector_type(8)));
+typedef float hl_f32x16_t __attribute__((ext_vector_type(16)));
+
+__global__ __launch_bounds__(256) void head_linear_mfma_kernel(
+        const bf16_t* __restrict__ x, int x_stride, int x_head, const bf16_t* __restrict__ w, bf16_t* __restrict__ out, int out_stride,
+        int out_head, int Tn, int N, int K, int wide, HeadExtra<bf16_t> extra) {
+    const int h = blockIdx.z, n0 = blockIdx.y * 64, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int t0 = blockIdx.x * 128 + wave * 32;
+    if (n0 >= N) {                                     // the blocks of the tail (there are none without one)
+        for (int e = threadIdx.x; e < 128 * extra.tail; e += 256) {
+            const int t = blockIdx.x * 128 + e / extra.tail, j = e % extra.tail;
+            if (t < Tn) st_f32(out + (size_t)t * out_stride + h * out_head + N + j, extra.turned(x + (size_t)t * x_stride + h * x_head + K, t, j));
+        }
+        return;
+    }
+    if (t0 >= Tn) return;
+    const int lr = lane & 31, lh = lane >> 5;
+    const int t = t0 + lr;
+    const bf16_t* xr = x + (size_t)min(t, Tn - 1) * x_stride + (size_t)h * x_head;
+    const bf16_t* w0 = w + ((size_t)h * N + min(n0 + lr, N - 1)) * K, *w1 = w + ((size_t)h * N + min(n0 + 32 + lr, N - 1)) * K;
+    hl_f32x16_t a0, a1;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) a0[i] = a1[i] = 0.f;
+    const hl_bf16x8_t zero = __builtin_bit_cast(hl_bf16x8_t, ri_u32x4_t{0u, 0u, 0u, 0u});
+#pragma unroll 4
+    for (int k0 = 0; k0 < K; k0 += 16) {
+        const int k = k0 + 8 * lh, kk = min(k, K - 8);
+        hl_bf16x8_t xv = *reinterpret_cast<const hl_bf16x8_t*>(xr + kk);
+        hl_bf16x8_t wa = *reinterpret_cast<const hl_bf16x8_t*>(w0 + kk), wb = *reinterpret_cast<const hl_bf16x8_t*>(w1 + kk);
+        if (k >= K) xv = wa = wb = zero;               // the upper half of a last step of eight
+        a0 = __builtin_amdgcn_mfma_f32_32x32x16_bf16(wa, xv, a0, 0, 0, 0);
+        a1 = __builtin_amdgcn_mfma_f32_32x32x16_bf16(wb, xv, a1, 0, 0, 0);
+    }
+    if (t >= Tn) return;
+    bf16_t* o = out + (size_t)t * out_stride + h * out_head;
+#pragma unroll
+    for (int tile = 0; tile < 2; ++tile)
+#pragma unroll
+        for (int i = 0; i < 16; i += 4) {              // registers i .. i + 3: outputs 8 (i / 4) + 4 lh + 0..3 of the tile
+            const int n = n0 + 32 * tile + 2 * i + 4 * lh;
+            float v[4];
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[e] = n + e < N ? extra.gated(tile == 0 ? a0[i + e] : a1[i + e], t, h * N + n + e) : 0.f;
+            if (wide && n + 4 <= N) VecLoad<4>::st(o + n, v);
+            else {
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                    if (n + e < N) st_f32(o + n + e, v[e]);
+            }
+        }
 }
 
 }  // namespace
@@ -308,15 +458,32 @@ extern "C" int ri_head_norm_kv_write(
                              "ri_head_norm_kv_write: no keys, values or cache given, or their row strides too small");
     if (T == 0) return 0;
     RI_REQUIRE(q && positions && row_of_token, "ri_head_norm_kv_write: null pointer");
+#define RI_HN(KERNEL, TT, GRID) KERNEL<<<GRID, 256, 0, stream>>>((TT*)q, q_stride, (const TT*)k, k_stride, (const TT*)v, v_stride, H, Hkv, dk, dv, qw, kw, do_norm, eps, \
+        temp_coef, temp_every, positions, row_of_token, (TT*)kc, (TT*)vc, table, max_blocks, page, write_kv, maps, rot, cos_t, sin_t)
+    if (dk % 8 == 0 && dk <= 256 && rot % 16 == 0 && q_stride % 8 == 0 && (!write_kv || k_stride % 8 == 0) && (uintptr_t)q % 16 == 0 &&
+        (!write_kv || ((uintptr_t)k % 16 == 0 && (uintptr_t)kc % 16 == 0)) && (uintptr_t)qw % 16 == 0 && (uintptr_t)kw % 16 == 0 &&
+        (uintptr_t)cos_t % 16 == 0 && (uintptr_t)sin_t % 16 == 0 && (dtype == RI_F32 || dtype == RI_BF16)) {
+        int lph = 1;
+        while (8 * lph < dk) lph *= 2;
+        const int hpb = 256 / lph;
+        const dim3 vgrid(T, T <= 256 ? min(((H + Hkv) * maps + hpb - 1) / hpb, 64) : 1);
+#define RI_HN_L(TT) do { if (lph == 1) RI_HN((head_norm_kv_write_vec_kernel<TT, 1>), TT, vgrid); else if (lph == 2) RI_HN((head_norm_kv_write_vec_kernel<TT, 2>), TT, vgrid); \
+        else if (lph == 4) RI_HN((head_norm_kv_write_vec_kernel<TT, 4>), TT, vgrid); else if (lph == 8) RI_HN((head_norm_kv_write_vec_kernel<TT, 8>), TT, vgrid); \
+        else if (lph == 16) RI_HN((head_norm_kv_write_vec_kernel<TT, 16>), TT, vgrid); else RI_HN((head_norm_kv_write_vec_kernel<TT, 32>), TT, vgrid); } while (0)
+        if (dtype == RI_F32) RI_HN_L(float);
+        else RI_HN_L(bf16_t);
+#undef RI_HN_L
+        RI_LAUNCHED("ri_head_norm_kv_write");
+        return 0;
+    }
     // a step of few tokens: a block for every four heads, so that no wave walks a chain of heads
     const int by = T <= 256 ? min(((H + Hkv) * maps + 3) / 4, 64) : 1;
     const dim3 grid(T, by);
-    if (dtype == RI_F32)
-        head_norm_kv_write_kernel<float><<<grid, 256, 0, stream>>>((float*)q, q_stride, (const float*)k, k_stride, (const float*)v, v_stride, H, Hkv, dk, dv, qw, kw, do_norm, eps, temp_coef, temp_every, positions, row_of_token, (float*)kc, (float*)vc, table, max_blocks, page, write_kv, maps, rot, cos_t, sin_t);
-    else if (dtype == RI_BF16)
-        head_norm_kv_write_kernel<bf16_t><<<grid, 256, 0, stream>>>((bf16_t*)q, q_stride, (const bf16_t*)k, k_stride, (const bf16_t*)v, v_stride, H, Hkv, dk, dv, qw, kw, do_norm, eps, temp_coef, temp_every, positions, row_of_token, (bf16_t*)kc, (bf16_t*)vc, table, max_blocks, page, write_kv, maps, rot, cos_t, sin_t);
+    if (dtype == RI_F32) RI_HN(head_norm_kv_write_kernel<float>, float, grid);
+    else if (dtype == RI_BF16) RI_HN(head_norm_kv_write_kernel<bf16_t>, bf16_t, grid);
     else
         return ri_fail("ri_head_norm_kv_write: unknown dtype %d", dtype);
+#undef RI_HN
     RI_LAUNCHED("ri_head_norm_kv_write");
     return 0;
 }
@@ -338,9 +505,9 @@ extern "C" int ri_latent_kv_write(
     RI_REQUIRE((!q || q_abs) && down && positions && row_of_token, "ri_latent_kv_write: null pointer");
     RI_REQUIRE(!ql || (ql_out && Rq > 0 && ql_stride >= Rq && qo_stride >= Rq), "ri_latent_kv_write: the queries' latent needs a place and row strides of at least its size");
     if (dtype == RI_F32)
-        latent_kv_write_kernel<float><<<T, 256, 0, stream>>>((const float*)q, q_stride, (const float*)down, down_stride, (float*)q_abs, qa_stride, H, d, r, R, rot, cw, eps, cos_t, sin_t, positions, row_of_token, (float*)kc, (float*)vc, table, max_blocks, page, write_kv, (const float*)ql, ql_stride, Rq, qlw, (float*)ql_out, qo_stride);
+        latent_kv_write_kernel<float><<<dim3(T, ql ? 2 : 1), 256, 0, stream>>>((const float*)q, q_stride, (const float*)down, down_stride, (float*)q_abs, qa_stride, H, d, r, R, rot, cw, eps, cos_t, sin_t, positions, row_of_token, (float*)kc, (float*)vc, table, max_blocks, page, write_kv, (const float*)ql, ql_stride, Rq, qlw, (float*)ql_out, qo_stride);
     else if (dtype == RI_BF16)
-        latent_kv_write_kernel<bf16_t><<<T, 256, 0, stream>>>((const bf16_t*)q, q_stride, (const bf16_t*)down, down_stride, (bf16_t*)q_abs, qa_stride, H, d, r, R, rot, cw, eps, cos_t, sin_t, positions, row_of_token, (bf16_t*)kc, (bf16_t*)vc, table, max_blocks, page, write_kv, (const bf16_t*)ql, ql_stride, Rq, qlw, (bf16_t*)ql_out, qo_stride);
+        latent_kv_write_kernel<bf16_t><<<dim3(T, ql ? 2 : 1), 256, 0, stream>>>((const bf16_t*)q, q_stride, (const bf16_t*)down, down_stride, (bf16_t*)q_abs, qa_stride, H, d, r, R, rot, cw, eps, cos_t, sin_t, positions, row_of_token, (bf16_t*)kc, (bf16_t*)vc, table, max_blocks, page, write_kv, (const bf16_t*)ql, ql_stride, Rq, qlw, (bf16_t*)ql_out, qo_stride);
     else
         return ri_fail("ri_latent_kv_write: unknown dtype %d", dtype);
     RI_LAUNCHED("ri_latent_kv_write");
@@ -364,13 +531,23 @@ extern "C" int ri_head_linear(const void* x, int x_stride, int x_head, const voi
         const dim3 few((N + 31) / 32 + (tail > 0), H);
         const int vl = dtype == RI_F32 ? 4 : 8;
         const bool vec = K % vl == 0 && x_stride % vl == 0 && x_head % vl == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)w % 16 == 0;
-#define RI_HLF(TT, VV) head_linear_few_kernel<TT, VV><<<few, 256, 0, stream>>>((const TT*)x, x_stride, x_head, (const TT*)w, (TT*)out, out_stride, out_head, T, N, K, \
-                                      HeadExtra<TT>{tail, rot, table_rows, cos_t, sin_t, positions, (const TT*)gate, gate_stride})
-        if (dtype == RI_F32) { if (vec) RI_HLF(float, true); else RI_HLF(float, false); }
-        else if (dtype == RI_BF16) { if (vec) RI_HLF(bf16_t, true); else RI_HLF(bf16_t, false); }
+#define RI_HLF(TY, VV, TT) head_linear_few_kernel<TY, VV, TT><<<few, 256, 0, stream>>>((const TY*)x, x_stride, x_head, (const TY*)w, (TY*)out, out_stride, out_head, T, N, K, \
+                                          HeadExtra<TY>{tail, rot, table_rows, cos_t, sin_t, positions, (const TY*)gate, gate_stride})
+#define RI_HLF_T(TY, VV) do { if (T <= 1) RI_HLF(TY, VV, 1); else if (T <= 2) RI_HLF(TY, VV, 2); else if (T <= 4) RI_HLF(TY, VV, 4); \
+                              else if (T <= 8) RI_HLF(TY, VV, 8); else RI_HLF(TY, VV, 16); } while (0)
+        if (dtype == RI_F32) { if (vec) RI_HLF_T(float, true); else RI_HLF_T(float, false); }
+        else if (dtype == RI_BF16) { if (vec) RI_HLF_T(bf16_t, true); else RI_HLF_T(bf16_t, false); }
         else
             return ri_fail("ri_head_linear: unknown dtype %d", dtype);
+#undef RI_HLF_T
 #undef RI_HLF
+        RI_LAUNCHED("ri_head_linear");
+        return 0;
+    }
+    if (dtype == RI_BF16 && K % 8 == 0 && x_stride % 8 == 0 && x_head % 8 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)w % 16 == 0) {
+        const int wide = out_stride % 4 == 0 && out_head % 4 == 0 && (uintptr_t)out % 8 == 0;
+        head_linear_mfma_kernel<<<dim3((T + 127) / 128, (N + 63) / 64 + (tail > 0), H), 256, 0, stream>>>((const bf16_t*)x, x_stride, x_head, (const bf16_t*)w,
+            (bf16_t*)out, out_stride, out_head, T, N, K, wide, HeadExtra<bf16_t>{tail, rot, table_rows, cos_t, sin_t, positions, (const bf16_t*)gate, gate_stride});
         RI_LAUNCHED("ri_head_linear");
         return 0;
     }

@@ -215,7 +215,8 @@ def load_part(part, seed, dtype, scale=1.0, replace=()):
 @pytest.mark.parametrize("H,G,dk,dv,scale,cap,dims,scaling", [
     (4, 2, 16, 24, 0.4, 3.0, 8, SCALING), (3, 3, 40, 36, 0.2, 50.0, 40, None), (8, 1, 32, 16, 0.3, 2.0, 2, None), (2, 2, 128, 128, 0.09, 5.0, 64, SCALING),
     (5, 5, 72, 200, 0.12, None, 30, None), (6, 1, 24, 40, 0.3, 1.0, 24, SCALING), (2, 1, 256, 256, 0.06, 8.0, 128, None), (1, 1, 6, 2, 0.8, 4.0, 4, None),
-    (32, 1, 8, 12, 0.5, 6.0, 8, None), (6, 2, 64, 128, 0.12, 20.0, 16, SCALING), (20, 1, 24, 72, 0.25, 3.0, 6, None), (3, 1, 10, 100, 0.5, 2.5, 10, None)])
+    (32, 1, 8, 12, 0.5, 6.0, 8, None), (6, 2, 64, 128, 0.12, 20.0, 16, SCALING), (20, 1, 24, 72, 0.25, 3.0, 6, None), (3, 1, 10, 100, 0.5, 2.5, 10, None),
+    (6, 3, 48, 40, 0.2, 4.0, 32, SCALING), (2, 1, 200, 24, 0.1, 6.0, 176, None), (5, 1, 8, 16, 0.5, 3.0, 4, None)])
 def test_capped_attention_alone(dtype, H, G, dk, dv, scale, cap, dims, scaling, portion_kernel):
     d, m = 48, att(H, G, dk, dv, scale, cap, dims, 50.0, scaling)
     part, pes = attention_part(d, m)
@@ -390,7 +391,8 @@ def test_capped_scores_and_weights_keep_their_32_bits(monkeypatch):
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("T", [1, 5, 16, 17, 70, 131])
-@pytest.mark.parametrize("H,N,K,tail,rot", [(3, 20, 8, 6, 4), (2, 64, 32, 16, 16), (5, 70, 13, 3, 2), (1, 33, 40, 5, 0), (4, 128, 64, 0, 0)])
+@pytest.mark.parametrize("H,N,K,tail,rot", [(3, 20, 8, 6, 4), (2, 64, 32, 16, 16), (5, 70, 13, 3, 2), (1, 33, 40, 5, 0), (4, 128, 64, 0, 0),
+                                            (3, 33, 24, 8, 4), (2, 100, 40, 8, 8), (3, 7, 8, 0, 0)])
 def test_head_product_with_tail_and_gate(dtype, T, H, N, K, tail, rot):
     from rustinfer_amd.kernels import ops
     dt = getattr(torch, dtype)
